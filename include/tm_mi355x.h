@@ -505,9 +505,10 @@ int tm_gemm_export(const char* path);
  * Norms, attention scores and weights, and the residual sum are fp32 in both.
  * Weight slots (tm_engine_weight_copy, checkpoint bytes: bf16, [out][in]): "embed", "l<i>.norm1", "l<i>.norm2" (with an ff),
  * "l<i>.mix.q|k|v|o", "l<i>.mix.sink" (with a sink), "l<i>.mlp.up|down", "final.norm", "head". */
-enum { TM_MIXER_ATTENTION = 1, TM_MIXER_LATENT = 2, TM_MIXER_LIGHTNING = 3, TM_MIXER_DELTA = 4, TM_MIXER_PARALLEL = 5, TM_MIXER_FORGET = 6 };
+enum { TM_MIXER_ATTENTION = 1, TM_MIXER_LATENT = 2, TM_MIXER_LIGHTNING = 3, TM_MIXER_DELTA = 4, TM_MIXER_PARALLEL = 5, TM_MIXER_FORGET = 6,
+       TM_MIXER_RETENTION = 7 };
 enum { TM_MLP_NONE = 0, TM_MLP_DENSE = 1, TM_MLP_GATED = 2, TM_MLP_MOE = 3 };
-enum { TM_ACT_RELU2 = 0, TM_ACT_GELU_TANH = 1, TM_ACT_SILU = 2, TM_ACT_XIELU = 3, TM_ACT_POLYNORM = 4 };
+enum { TM_ACT_RELU2 = 0, TM_ACT_GELU_TANH = 1, TM_ACT_SILU = 2, TM_ACT_XIELU = 3, TM_ACT_POLYNORM = 4, TM_ACT_CLAMPED = 5 };
 enum { TM_DTYPE_BF16 = 0, TM_DTYPE_F32 = 1 };
 /* Further block forms, mixers and feed-forwards (every switch off at 0: the block above):
  *   one_norm:    both sublayers read norm1(x) (no norm2)
@@ -608,6 +609,24 @@ typedef struct tm_layer_spec {
      *   TM_ACT_POLYNORM ("mlp.act" = [a, b, c, e]): act(z) = a N(z) + b N(z^2) + c N(z^3) + e, N(v) = v / sqrt(mean(v^2) + norm_eps) over the ff values
      *     of a token. */
     int          pre_norm, q_rank, kv_from;
+    /* both_norms blocks (off at 0): x <- x + N1b(mixer(N1 x)); x <- x + N2b(ff(N2 x)), N the model's RMS norm (norm_offset + "norm<i>", "norm<i>b");
+     * an RMS norm ends the model.  loop_pass > 0 with tm_layered_config.loop_add: the embedding output joins the stream ahead of this run.
+     *   TM_MIXER_RETENTION: S <- decay[head] S + k v^T, o = S^T q per head; queries and keys turn in their first rot_dims channels (channel i with
+     *     i + rot_dims / 2), keys then times dim^-1/2; every head's o to unit RMS, times silu("mix.g" h); then "mix.o".
+     *   TM_MIXER_PARALLEL in such a block: left_scale * left + right_scale * right of the same input.
+     *     left ("mix.left.*", sizes heads / kv_heads / dim / vdim): conv_taps, rotation as above, scale, softcap, window, sink ("sink" [heads]).
+     *     right ("mix.right.*", sizes r_heads / r_dim, r_vdim = r_dim): with h' the previous token's input (zeros ahead of the sequence) each
+     *       projection s of r, k, v, g, w reads h + (h' - h) * "mu.<s>"; decay w = exp(-exp("w2" tanh("w1" .) + "w0")) per head and key channel;
+     *       o = (S + diag("u") k v^T)^T r, then S <- diag(w) S + k v^T; every head's o to unit RMS, times "norm", times silu("g" .); then "o".
+     *       decay_rank = rows of "w1".  h' is part of the slot's state.
+     *   TM_MLP_GATED with TM_ACT_CLAMPED: g = min(gate h, act_limit), u = clamp(up h, -act_limit, act_limit), down(g sigmoid(act_alpha g) (u + 1)).
+     *   TM_MLP_MOE: gated experts with act; scores s = sigmoid("mlp.router" h); experts are ordered by s + "mlp.correction" (router_correction) and
+     *     come from the group_keep best of group_count equal groups (a group counts the sum of its two best); the chosen scores (divided by
+     *     their sum with router_renorm) weight the experts' OUTPUTS; a shared expert ("mlp.shared.gate|up|down", shared_ff) is added, times
+     *     sigmoid("mlp.shared.sg" h) with shared_gate. */
+    int   both_norms;
+    float left_scale, right_scale, act_limit, act_alpha;
+    int   group_count, group_keep, router_correction, router_renorm, shared_gate;
 } tm_layer_spec;
 typedef struct tm_layered_config {
     int                  width, vocab, n_layers;
@@ -625,6 +644,8 @@ typedef struct tm_layered_config {
      *     [width][side_dim], "l<i>.side.norm" [width])
      *   depth_avg: what layer i hands on is sum_j "l<i>.dwa"[j] X_j, j = 0 .. i + 1, X_0 the embedding output, X_(j + 1) the result of layer j */
     int                  side_dim, depth_avg;
+    int                  loop_add;  /* != 0: the embedding output is added to the stream ahead of every layer run with loop_pass > 0 */
+    int                  tied_head; /* != 0: the logits come from the embedding table, no "head" */
 } tm_layered_config;
 /* cfg->model is ignored; tp must be 1; quant_policy 0 (the cache holds the activation type) */
 int tm_engine_create_layered(tm_engine** out, const tm_engine_config* cfg, const tm_layered_config* model);

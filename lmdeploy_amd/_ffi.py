@@ -81,7 +81,9 @@ class LayerSpec(C.Structure):
                 ('yarn_factor', c_float), ('yarn_original', c_float), ('yarn_fast', c_float), ('yarn_slow', c_float),
                 ('dist_buckets', c_int), ('dist_max', c_float), ('r_heads', c_int), ('r_kv_heads', c_int), ('r_dim', c_int),
                 ('r_vdim', c_int), ('r_conv', c_int), ('a_rank', c_int), ('g_rank', c_int), ('pre_norm', c_int), ('q_rank', c_int),
-                ('kv_from', c_int)]
+                ('kv_from', c_int), ('both_norms', c_int), ('left_scale', c_float), ('right_scale', c_float), ('act_limit', c_float),
+                ('act_alpha', c_float), ('group_count', c_int), ('group_keep', c_int), ('router_correction', c_int),
+                ('router_renorm', c_int), ('shared_gate', c_int)]
 
 
 class LayeredConfig(C.Structure):
@@ -89,7 +91,7 @@ class LayeredConfig(C.Structure):
     _fields_ = [('width', c_int), ('vocab', c_int), ('n_layers', c_int), ('layers', POINTER(LayerSpec)), ('norm_eps', c_float),
                 ('norm_offset', c_float), ('residual_mult', c_float), ('logit_scale', c_float), ('dtype', c_int), ('loop_times', c_int),
                 ('final_layer_norm', c_int), ('embed_scale', c_float), ('logit_softcap', c_float), ('norm_groups', c_int),
-                ('side_dim', c_int), ('depth_avg', c_int)]
+                ('side_dim', c_int), ('depth_avg', c_int), ('loop_add', c_int), ('tied_head', c_int)]
 
 
 class StepEntry(C.Structure):

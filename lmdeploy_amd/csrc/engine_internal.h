@@ -123,6 +123,18 @@ struct LmLayer {
     DenseWeight  uq;                           // queries from their latent
     float *      cq_norm = nullptr, *f_bias = nullptr, *f_low = nullptr;
     DenseWeight  side_gate, side_proj;         // the layer's part of the token-side table: gate and projection back to the width
+    // blocks with a norm on both sides of each sublayer (spec.both_norms): x += N1b(mixer(N1 x)); x += N2b(ff(N2 x)).  `qkv` columns (fp32 output)
+    //   retention: [q | k | v | gate]
+    //   parallel:  [left q | left k | left v] of the row, then r, k, v, gate and the decay's inner part, each of its own mix of the row and its
+    //              predecessor (a segment of the product, starting at a multiple of 128: seg_n0)
+    // `wo` closes both mixers of the parallel pair over [left heads | right heads]; `router` holds the shared expert's gate behind the logits
+    bool         both = false;
+    int          seg_n0[kDenseMaxSeg] = {}, n_seg = 0;
+    int          c_rr = 0;                     // parallel: the right mixer's query column (keys c_rk, values c_rv, gate c_rg, decay c_w1)
+    int          c_rg = 0;
+    float *      norm1b = nullptr, *norm2b = nullptr, *mu = nullptr, *bonus = nullptr, *correction = nullptr;
+    size_t       shift_offset = 0;             // the previous token's input inside a slot of the state pool
+    DenseWeight  sh_gu;                        // a shared expert larger than the routed ones: its [gate | up]
     float *      side_w = nullptr, *dwa = nullptr;  // ... its norm; weights of the depth average [layer + 2]
 };
 
@@ -157,6 +169,11 @@ struct LayeredModel {
     // pre-norm models: normed query latents, token-side activations, the second embedding table (bf16), and the results of the layers so
     // far, [n_layers][max_tokens][width] fp32 (entry 0: the embedding output), for the average over the depth
     bool                 has_pre = false;
+    // models with norms on both sides of a sublayer: a parallel pair's inputs, [row | its mixes] per row, and the normed rows in fp32
+    bool                 has_both = false;
+    void*                d_mix = nullptr;
+    int                  ldmixin = 0;
+    float*               d_hf = nullptr;
     void *               d_cq = nullptr, *d_side = nullptr, *side_embed = nullptr;
     int                  ldcq = 0, ldside = 0;
     float*               d_hist = nullptr;

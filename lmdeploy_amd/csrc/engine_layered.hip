@@ -53,6 +53,18 @@
 //   h        = LN2 x;  z = h . Wup^T (fp32);  a = PolyNorm(z);  x += a . Wdown^T, h = x in the activation type      (one epilogue)
 //   g        = gelu(h . gate^T) * side_embed[token]                GEMM epilogue;   y = g . proj^T
 //   x        = sum_j dwa[j] X_j, X_(i+1) = x + RMS(y) w;  h = LN1 of the next layer                                 one launch (launch_layer_close)
+//
+// Blocks with a norm on both sides of each sublayer (LmLayer::both): x += N1b(mixer(N1 x)); x += N2b(ff(N2 x)), RMS norms,
+//   h        = N1 x                                                (written by the previous layer's closing launch; a parallel pair's mixes of
+//              the row and its predecessor too, for decoded tokens; prompt portions form them in launch_token_shift)
+//   retention:  proj = h . [q | k | v | gate]^T -> launch_state_mix (rotation inside) -> unit RMS per head, silu gate
+//   parallel:   proj = ONE segmented product over [h | mixes] -> left: convolution, launch_attn_prep (rotation; values times left_scale), attention
+//               with window, cap and sink -> cat[:, 0 : heads vdim];  right: decay's outer product -> launch_state_mix -> head norm, silu gate,
+//               times right_scale -> cat[:, heads vdim :]
+//   y        = cat . Wo^T (both mixers in one sum);  x += N1b y, h = N2 x                                             one launch (launch_block_close)
+//   dense:   y = down(clamped pair);   experts: grouped router -> rows sorted by expert (+ all rows for a shared expert no larger than they) ->
+//            two batched products -> weighted sum + gated shared expert
+//   x       += N2b y (+ x0 where the next run opens a later pass of a loop), h = N1 of the next layer                 one launch (launch_block_close)
 #include "engine_internal.h"
 
 namespace tmk {
@@ -405,6 +417,100 @@ static int process_group_layer(tm_engine* e, int i, LmLayer& L, int dt)
     return 0;
 }
 
+// [gate | up] pair and down matrix of a gated feed-forward "<pre>gate|up|down" -> item `x` of the images
+static int place_gated(tm_engine* e, DenseWeight& gu, DenseWeight& down, int i, const std::string& pre, int ff, int x)
+{
+    const int W = e->lm->cfg.width;
+    TM_TRY(place(e, gu, 0, 0, lname(i, (pre + "gate").c_str()), ff, W, 0, x, false, 1));
+    TM_TRY(place(e, gu, 0, 0, lname(i, (pre + "up").c_str()), ff, W, 0, x, false, 2));
+    return place(e, down, 0, 0, lname(i, (pre + "down").c_str()), W, ff, 0, x);
+}
+
+// blocks with a norm on both sides of each sublayer (see the head of this file)
+static int process_both_layer(tm_engine* e, int i, LmLayer& L, int dt)
+{
+    const tm_layer_spec& s = L.spec;
+    const int            W = e->lm->cfg.width, H = s.heads;
+    hipStream_t          st = e->stream;
+    TM_TRY(to_f32(e, lname(i, "norm1"), W, &L.norm1));
+    TM_TRY(to_f32(e, lname(i, "norm1b"), W, &L.norm1b));
+    TM_TRY(dense_weight_alloc(L.qkv, W, L.c_end, dt, st));
+    if (s.rot_dims > 0) {
+        TM_TRY(upload_f32(e, rotation_frequencies(s), &L.inv_freq));
+    }
+    if (s.mixer == TM_MIXER_RETENTION) {
+        TM_TRY(place(e, L.qkv, 0, 0, lname(i, "mix.q"), L.n_q, W));
+        TM_TRY(place(e, L.qkv, L.c_k, 0, lname(i, "mix.k"), L.n_k, W));
+        TM_TRY(place(e, L.qkv, L.c_v, 0, lname(i, "mix.v"), L.n_v, W));
+        TM_TRY(place(e, L.qkv, L.c_g, 0, lname(i, "mix.g"), L.n_att, W));
+        TM_TRY(upload_f32(e, L.decay_h, &L.decay_d));
+        TM_TRY(dense_weight_alloc(L.wo, L.n_att, W, dt, st));
+        TM_TRY(place(e, L.wo, 0, 0, lname(i, "mix.o"), W, L.n_att));
+    }
+    else {
+        const int n_r = L.r_nv;
+        TM_TRY(place(e, L.qkv, 0, 0, lname(i, "mix.left.q"), L.n_q, W));
+        TM_TRY(place(e, L.qkv, L.c_k, 0, lname(i, "mix.left.k"), L.n_k, W));
+        TM_TRY(place(e, L.qkv, L.c_v, 0, lname(i, "mix.left.v"), L.n_v, W));
+        if (s.conv_taps > 0) {
+            TM_TRY(dmalloc(&L.conv_w, (size_t)L.conv_ch * s.conv_taps));
+            TM_TRY(to_f32_at(e, lname(i, "mix.left.q.conv"), (size_t)L.n_q * s.conv_taps, L.conv_w));
+            TM_TRY(to_f32_at(e, lname(i, "mix.left.k.conv"), (size_t)L.n_k * s.conv_taps, L.conv_w + (size_t)L.c_k * s.conv_taps));
+            TM_TRY(to_f32_at(e, lname(i, "mix.left.v.conv"), (size_t)L.n_v * s.conv_taps, L.conv_w + (size_t)L.c_v * s.conv_taps));
+        }
+        if (s.sink) {
+            TM_TRY(to_f32(e, lname(i, "mix.left.sink"), H, &L.sink));
+        }
+        TM_TRY(dmalloc(&L.mu, (size_t)5 * W));
+        const char* mixes[5] = {"r", "k", "v", "g", "w"};
+        const int   cols[5]  = {L.c_rr, L.c_rk, L.c_rv, L.c_rg, L.c_w1};
+        for (int j = 0; j < 5; ++j) {
+            const std::string leaf = mixes[j];
+            TM_TRY(to_f32_at(e, lname(i, ("mix.right.mu." + leaf).c_str()), W, L.mu + (size_t)j * W));
+            TM_TRY(place(e, L.qkv, cols[j], 0, lname(i, ("mix.right." + (j == 4 ? "w1" : leaf)).c_str()), j == 4 ? s.decay_rank : n_r, W));
+        }
+        TM_TRY(dense_weight_alloc(L.w2, s.decay_rank, n_r, dt, st));
+        TM_TRY(place(e, L.w2, 0, 0, lname(i, "mix.right.w2"), n_r, s.decay_rank));
+        TM_TRY(to_f32(e, lname(i, "mix.right.w0"), n_r, &L.w0));
+        TM_TRY(to_f32(e, lname(i, "mix.right.u"), n_r, &L.bonus));
+        TM_TRY(to_f32(e, lname(i, "mix.right.norm"), n_r, &L.r_norm));
+        TM_TRY(dense_weight_alloc(L.wo, L.n_att + n_r, W, dt, st));
+        TM_TRY(place(e, L.wo, 0, 0, lname(i, "mix.left.o"), W, L.n_att));
+        TM_TRY(place(e, L.wo, 0, L.n_att, lname(i, "mix.right.o"), W, n_r));
+    }
+    if (s.mlp == TM_MLP_NONE) {
+        return 0;
+    }
+    TM_TRY(to_f32(e, lname(i, "norm2"), W, &L.norm2));
+    TM_TRY(to_f32(e, lname(i, "norm2b"), W, &L.norm2b));
+    const int items = s.mlp == TM_MLP_MOE ? s.experts + (L.shared_fused ? 1 : 0) : 1;
+    TM_TRY(dense_weight_alloc(L.gu, W, dense_pair_rows(s.ff), dt, st, items));  // gate and up interleaved: the activation is the GEMM's epilogue
+    TM_TRY(dense_weight_alloc(L.down, s.ff, W, dt, st, items));
+    if (s.mlp == TM_MLP_GATED) {
+        return place_gated(e, L.gu, L.down, i, "mlp.", s.ff, 0);
+    }
+    for (int x = 0; x < s.experts; ++x) {
+        TM_TRY(place_gated(e, L.gu, L.down, i, "mlp.e" + std::to_string(x) + ".", s.ff, x));
+    }
+    TM_TRY(dense_weight_alloc(L.router, W, s.experts + (s.shared_gate ? 1 : 0), dt, st));
+    TM_TRY(place(e, L.router, 0, 0, lname(i, "mlp.router"), s.experts, W));
+    if (s.shared_gate) {
+        TM_TRY(place(e, L.router, s.experts, 0, lname(i, "mlp.shared.sg"), 1, W));
+    }
+    if (s.router_correction) {
+        TM_TRY(to_f32(e, lname(i, "mlp.correction"), s.experts, &L.correction));
+    }
+    if (L.shared_fused) {  // zero-padded to the routed experts' size
+        TM_TRY(place_gated(e, L.gu, L.down, i, "mlp.shared.", s.shared_ff, s.experts));
+    }
+    else if (s.shared_ff > 0) {
+        TM_TRY(dense_weight_alloc(L.sh_gu, W, dense_pair_rows(s.shared_ff), dt, st));
+        TM_TRY(dense_weight_alloc(L.sh_down, s.shared_ff, W, dt, st));
+        TM_TRY(place_gated(e, L.sh_gu, L.sh_down, i, "mlp.shared.", s.shared_ff, 0));
+    }
+    return 0;
+}
+
 // pre-norm blocks (see the head of this file)
 static int process_pre_layer(tm_engine* e, int i, LmLayer& L, int dt)
 {
@@ -572,6 +678,10 @@ int layered_process_weights(tm_engine* e)
             continue;
         }
         const tm_layer_spec& s = L.spec;
+        if (L.both) {
+            TM_TRY(process_both_layer(e, i, L, dt));
+            continue;
+        }
         if (L.pre) {
             TM_TRY(process_pre_layer(e, i, L, dt));
             continue;
@@ -604,7 +714,12 @@ int layered_process_weights(tm_engine* e)
     }
     for (int i = 0; i < c.n_layers; ++i) {  // borrowed weights
         LmLayer& L = lm.layers[i];
-        if (L.src != i) {
+        if (L.src != i && L.both) {  // equal in everything but the run's own spec; cache and state places are given out later
+            LmLayer B = lm.layers[L.src];
+            B.spec = L.spec, B.src = L.src;
+            L      = B;
+        }
+        else if (L.src != i) {
             const LmLayer& S = lm.layers[L.src];
             L.qkv = S.qkv, L.up = S.up, L.out = S.out, L.norm1 = S.norm1, L.norm2 = S.norm2, L.sink = S.sink;
             L.wo = S.wo, L.gu = S.gu, L.down = S.down, L.uk = S.uk, L.uv = S.uv;
@@ -620,7 +735,7 @@ int layered_process_weights(tm_engine* e)
         TM_TRY(to_f32(e, "loop.step", (size_t)c.loop_times * W, &lm.loop_step));
     }
     TM_TRY(dense_weight_alloc(lm.head, W, c.vocab, dt, e->stream));
-    TM_TRY(place(e, lm.head, 0, 0, "head", c.vocab, W));
+    TM_TRY(place(e, lm.head, 0, 0, c.tied_head ? "embed" : "head", c.vocab, W));
     TM_TRY(to_f32(e, "final.norm", W, &lm.final_norm));
     if (c.final_layer_norm && c.norm_groups == 0) {
         TM_TRY(to_f32(e, "final.norm.b", W, &lm.final_norm_b));
@@ -674,7 +789,8 @@ int layered_init_synthetic(tm_engine* e, uint64_t seed)
         const bool          join = leaf == "out" && (n.find("left.out") != std::string::npos || n.find("right.out") != std::string::npos);
         const bool          vec = isnorm || join || leaf == "sink" || leaf == "r1" || leaf == "r2" || (leaf == "b" && n.find("right.b") == std::string::npos)
                                   || leaf == "step" || leaf == "w0" || leaf == "act" || leaf == "lq1" || leaf == "lk1" || leaf == "lq2" || leaf == "lk2"
-                                  || leaf == "rel" || leaf == "A_log" || leaf == "dt_bias" || leaf == "lower" || leaf == "dwa";
+                                  || leaf == "rel" || leaf == "A_log" || leaf == "dt_bias" || leaf == "lower" || leaf == "dwa" || leaf == "u"
+                                  || leaf == "correction" || n.find(".mu.") != std::string::npos;
         // matrices: N(0, 1 / in_features) keeps every projection's output at the scale of its input; vectors: small, around zero (norm
         // weights around 1 - norm_offset; distance-penalty numbers positive)
         float stdv = 0.02f, mean = 0.f;
@@ -684,8 +800,14 @@ int layered_init_synthetic(tm_engine* e, uint64_t seed)
         else if (leaf == "r1" || leaf == "r2") {
             mean = 0.5f;
         }
-        else if (leaf == "lower") {
+        else if (leaf == "lower" || n.find(".mu.") != std::string::npos) {
             mean = 0.5f;
+        }
+        else if (leaf == "w0" && n.find("right.w0") != std::string::npos) {  // states that hold for some tens of tokens
+            mean = -3.f;
+        }
+        else if (leaf == "norm" && n.find("right.norm") != std::string::npos) {
+            mean = 1.f;  // (not stored around zero)
         }
         else if (leaf == "dwa") {  // an even average
             mean = 1.f / (float)cnt;
@@ -751,13 +873,18 @@ int layered_start(tm_engine* e)
             L.state_floats = parallel ? state_mix_floats(L.spec.r_heads, L.spec.r_dim, L.spec.r_vdim) : state_mix_floats(L.spec.heads, L.spec.dim, L.spec.vdim);
             lm.state_slot_floats += L.state_floats;
             max_mix  = std::max(max_mix, parallel ? std::max(L.r_nv, L.spec.r_heads * L.spec.r_dim) : L.n_att);
-            max_lora = std::max(max_lora, parallel ? L.lora_g1 + L.g2.Kp : L.w2.Kp);
+            max_lora = std::max(max_lora, parallel && !L.both ? L.lora_g1 + L.g2.Kp : L.w2.Kp);
+        }
+        if (L.n_seg > 1) {  // the previous token's input, at a multiple of four floats
+            L.shift_offset = lm.state_slot_floats = (lm.state_slot_floats + 3) / 4 * 4;
+            lm.state_slot_floats += m.width;
+            lm.ldmixin = std::max(lm.ldmixin, L.n_seg * lm.ldw);
         }
         if (L.conv_taps > 0) {  // the last taps - 1 inputs of a short convolution are state too
             L.conv_offset = lm.state_slot_floats;
             L.conv_floats = (size_t)(L.conv_taps - 1) * L.conv_ch;
             lm.state_slot_floats += L.conv_floats;
-            max_conv = std::max(max_conv, L.conv_ch + (parallel ? 2 * L.spec.r_heads * L.spec.r_dim : 0));
+            max_conv = std::max(max_conv, L.conv_ch + (parallel && !L.both ? 2 * L.spec.r_heads * L.spec.r_dim : 0));
         }
         if (L.pre && L.spec.kv_from >= 0) {  // another layer's entries
             L.kv_offset = lm.layers[L.spec.kv_from].kv_offset, L.v_offset = lm.layers[L.spec.kv_from].v_offset;
@@ -789,13 +916,17 @@ int layered_start(tm_engine* e)
             max_ff    = std::max(max_ff, L.down.Kp);
             lm.ldside = std::max(lm.ldside, L.side_proj.Kp);
             if (L.spec.mixer == TM_MIXER_FORGET) {
-                lm.blocks_floats = std::max(lm.blocks_floats, forget_workspace_floats((int)T, B, L.spec.heads, L.spec.dim));
+                lm.blocks_floats = std::max(lm.blocks_floats, decay_workspace_floats((int)T, B, L.spec.heads, L.spec.dim));
             }
             continue;
         }
-        if (L.post) {
+        if (L.both) {
+            lm.blocks_floats = std::max(lm.blocks_floats, parallel ? decay_workspace_floats((int)T, B, L.spec.r_heads, L.spec.r_dim)
+                                                                   : decay_workspace_floats((int)T, B, L.spec.heads, L.spec.dim));
+        }
+        if (L.post || L.both) {
             max_cat  = std::max(max_cat, L.wo.Kp);
-            max_proj = std::max(max_proj, std::max(L.qkv.N, L.spec.experts));
+            max_proj = std::max(max_proj, std::max(L.qkv.N, L.spec.experts + 1));
             max_q    = std::max(max_q, L.has_cache ? L.a_heads * L.a_dim : 0);
             if (L.spec.mlp) {
                 max_ff     = std::max(max_ff, std::max(L.down.Kp, L.sh_down.Kp));
@@ -848,6 +979,9 @@ int layered_start(tm_engine* e)
             TM_TRY(lm_alloc(&lm.d_offsets, (size_t)1026, st));
         }
     }
+    if (m.loop_add) {
+        TM_TRY(lm_alloc(&lm.d_x0, T * m.width, st));
+    }
     if (m.loop_times > 0) {
         lm.ld2w = lm.loop_in.Kp;
         TM_TRY(lm_alloc(&lm.d_x0, T * m.width, st));
@@ -870,6 +1004,26 @@ int layered_start(tm_engine* e)
             TM_TRY(lm_alloc(&lm.d_gate2, T * lm.ldmix, st));
         }
     }
+    if (lm.has_both) {
+        lm.ldmix  = std::max(4, (max_mix + 3) / 4 * 4);
+        lm.ldlora = std::max(32, max_lora);
+        TM_TRY(lm_alloc(&lm.d_y, T * m.width, st));
+        TM_TRY(lm_alloc(&lm.d_mixo, T * lm.ldmix, st));
+        TM_TRY(lm_alloc(&lm.d_blocks, lm.blocks_floats, st));
+        if (lm.ldmixin > 0) {
+            TM_TRY(lm_alloc((char**)&lm.d_mix, T * lm.ldmixin * lm.elem, st));
+            TM_TRY(lm_alloc(&lm.d_hf, T * m.width, st));
+            TM_TRY(lm_alloc(&lm.d_wdec, T * lm.ldmix, st));
+            TM_TRY(lm_alloc((char**)&lm.d_lora, T * lm.ldlora * lm.elem, st));
+        }
+        if (max_conv > 0) {
+            lm.ldconv = (max_conv + 3) / 4 * 4;
+            TM_TRY(lm_alloc(&lm.d_conv, T * lm.ldconv, st));
+        }
+        if (any_moe) {
+            TM_TRY(lm_alloc(&lm.d_y2, T * m.width, st));
+        }
+    }
     if (lm.has_pre) {
         if (max_mix > 0) {
             lm.ldmix = (max_mix + 3) / 4 * 4;
@@ -890,6 +1044,7 @@ int layered_start(tm_engine* e)
             TM_TRY(lm_alloc(&lm.d_hist, (size_t)m.n_layers * lm.hist_stride, st));
         }
     }
+    lm.state_slot_floats = (lm.state_slot_floats + 3) / 4 * 4;
     if (lm.state_slot_floats > 0) {
         TM_TRY(lm_alloc(&lm.d_state, ((size_t)B + 1) * lm.state_slot_floats, st));
     }
@@ -972,10 +1127,10 @@ void layered_free(tm_engine* e)
             dense_weight_free(L.wo), dense_weight_free(L.gu), dense_weight_free(L.down), dense_weight_free(L.uk), dense_weight_free(L.uv);
             dense_weight_free(L.w2), dense_weight_free(L.router), dense_weight_free(L.sh_up), dense_weight_free(L.sh_down);
             dense_weight_free(L.wo_r), dense_weight_free(L.a2), dense_weight_free(L.g2);
-            dense_weight_free(L.uq), dense_weight_free(L.side_gate), dense_weight_free(L.side_proj);
+            dense_weight_free(L.uq), dense_weight_free(L.side_gate), dense_weight_free(L.side_proj), dense_weight_free(L.sh_gu);
             for (float* p : {L.norm1, L.norm2, L.sink, L.r1, L.r2, L.rg1_b, L.rg2_b, L.c_norm, L.inv_freq, L.norm1_b, L.norm2_b, L.proj_bias,
                              L.q_w, L.k_w, L.mix_norm, L.w0, L.act_par, L.decay_d, L.conv_w, L.lambda, L.dist_tab, L.talk, L.zero_sink, L.join_l,
-                             L.join_r, L.a_log, L.dt_bias, L.r_norm, L.cq_norm, L.f_bias, L.f_low, L.side_w, L.dwa}) {
+                             L.join_r, L.a_log, L.dt_bias, L.r_norm, L.cq_norm, L.f_bias, L.f_low, L.side_w, L.dwa, L.norm1b, L.norm2b, L.mu, L.bonus, L.correction}) {
                 if (p) {
                     (void)hipFree(p);
                 }
@@ -985,7 +1140,8 @@ void layered_free(tm_engine* e)
     dense_weight_free(lm.head);
     dense_weight_free(lm.loop_in);
     for (void* p : {(void*)lm.d_y, (void*)lm.d_mixo, (void*)lm.d_aux, (void*)lm.d_wdec, lm.d_lora, (void*)lm.d_state, (void*)lm.final_norm_b,
-                    (void*)lm.d_y2, (void*)lm.d_conv, (void*)lm.d_gate2, lm.d_cq, lm.d_side, lm.side_embed, (void*)lm.d_hist, (void*)lm.d_blocks}) {
+                    (void*)lm.d_y2, (void*)lm.d_conv, (void*)lm.d_gate2, lm.d_cq, lm.d_side, lm.side_embed, (void*)lm.d_hist, (void*)lm.d_blocks,
+                    lm.d_mix, (void*)lm.d_hf}) {
         if (p) {
             (void)hipFree(p);
         }
@@ -1014,7 +1170,7 @@ static GeneralAttnParams attn_params(tm_engine* e, const LmLayer& L, const LmPar
     p.out          = (char*)lm.d_cat + (size_t)P.row0 * lm.ldcat * lm.elem;
     p.ldq          = lm.ldqkv;
     p.ldo          = lm.ldcat;
-    if (L.wide || L.post || L.pre) {
+    if (L.wide || L.post || L.pre || L.both) {
         p.q   = (const char*)lm.d_q + (size_t)P.row0 * lm.ldq * lm.elem;
         p.ldq = lm.ldq;
         if (L.spec.mixer == TM_MIXER_LATENT) {  // the attention output stays in the latent space until the value expansion
@@ -1511,6 +1667,183 @@ static int pre_layer(tm_engine* e, int li, const LmLayer& L, const LmLayer* next
     return 0;
 }
 
+// the rows and sequences whose token mixes a parallel pair reads, over the rows of a part
+static TokenShift token_shift_args(tm_engine* e, const LmLayer& L, const LmPart& P)
+{
+    LayeredModel& lm = *e->lm;
+    TokenShift    ts;
+    ts.n_mix = L.n_seg - 1, ts.mu = L.mu;
+    ts.out = (char*)lm.d_mix + (size_t)P.row0 * lm.ldmixin * lm.elem, ts.ld = lm.ldmixin, ts.mix_stride = lm.ldw, ts.elem_bytes = lm.elem;
+    ts.seqs              = state_seqs(e, P);
+    ts.seqs.layer_offset = L.shift_offset;
+    return ts;
+}
+
+// a sublayer's result (y, normed with post_w; nullptr: none yet) and the embedding output (x0; nullptr: not) join the stream; the norm next_w
+// (nullptr: none) becomes the next product's operand -- with the token mixes when `pair` (a parallel layer) is what reads it
+static int close_block(tm_engine* e, const float* y, const float* post_w, const float* x0, const float* next_w, const LmLayer* pair, int M,
+                       const LmPart* parts, int nparts)
+{
+    LayeredModel& lm = *e->lm;
+    BlockClose    bc;
+    bc.x = lm.d_res, bc.y = y, bc.post_w = post_w, bc.x0 = x0, bc.next_w = next_w, bc.w_offset = lm.cfg.norm_offset, bc.eps = lm.cfg.norm_eps;
+    bc.M = M, bc.H = lm.cfg.width, bc.h = lm.d_h1, bc.ldh = lm.ldw, bc.h_elem_bytes = lm.elem;
+    if (pair && pair->n_seg > 1) {
+        bc.h = lm.d_mix, bc.ldh = lm.ldmixin, bc.hf = lm.d_hf;
+        if (parts[0].decode) {  // (decoded tokens come first: their mixes need nothing but the slot's state)
+            bc.shift_rows = parts[0].rows;
+            bc.shift      = token_shift_args(e, *pair, parts[0]);
+        }
+    }
+    TM_PROF(P_RES_NORM, TM_TRY(launch_block_close(bc, e->stream)));
+    if (pair && pair->n_seg > 1) {
+        for (int i = 0; i < nparts; ++i) {
+            const LmPart& P = parts[i];
+            if (!P.decode) {
+                TM_PROF(P_RES_NORM, TM_TRY(launch_token_shift(lm.d_hf + (size_t)P.row0 * lm.cfg.width, token_shift_args(e, *pair, P), lm.d_row_seq + P.row0,
+                                                              lm.d_row_pos + P.row0, P.rows, lm.cfg.width, e->stream)));
+            }
+        }
+    }
+    return 0;
+}
+
+// routed experts with a grouped router and a gated shared expert over lm.d_h1 -> lm.d_y
+static int grouped_experts(tm_engine* e, const LmLayer& L, int M)
+{
+    LayeredModel&        lm = *e->lm;
+    const tm_layer_spec& s  = L.spec;
+    hipStream_t          st = e->stream;
+    const int            W = lm.cfg.width, k = s.top, E = s.experts;
+    TM_PROF(P_GEMM_GATE_UP, TM_TRY(launch_dense_linear(L.router, lm.d_h1, lm.ldw, lm.d_proj, lm.ldproj, M, kDenseScaleF32, 1.f, st)));
+    TM_PROF(P_GEMM_GATE_UP, TM_TRY(launch_moe_topk_grouped(lm.d_topk_ids, lm.d_topk_w, lm.d_proj, lm.ldproj, L.correction, M, E, std::max(1, s.group_count),
+                                                           std::max(1, s.group_keep), k, s.router_renorm != 0, st)));
+    TM_PROF(P_GEMM_GATE_UP, TM_TRY(launch_moe_route(lm.d_offsets, lm.d_f2n, lm.d_en2f, lm.d_topk_ids, M, E, k, st)));
+    TM_PROF(P_GEMM_GATE_UP, TM_TRY(launch_moe_gather(lm.d_moe_x, lm.ldw, lm.d_h1, lm.ldw, lm.elem, lm.d_topk_w, lm.d_en2f, M, W, k, false, st,
+                                                     L.shared_fused ? lm.d_offsets : nullptr, E)));
+    const int rows = M * (k + (L.shared_fused ? 1 : 0));
+    DenseCall c;
+    c.epi         = kDenseGatedAct;
+    c.act         = s.act;
+    c.n_out       = s.ff;
+    c.count       = E + (L.shared_fused ? 1 : 0);
+    c.row_offsets = lm.d_offsets;
+    TM_PROF(P_GEMM_GATE_UP, TM_TRY(launch_dense_call(L.gu, lm.d_moe_x, lm.ldw, lm.d_ff, lm.ldff, rows, c, st)));
+    c.epi = kDenseScaleF32;
+    TM_PROF(P_GEMM_DOWN, TM_TRY(launch_dense_call(L.down, lm.d_ff, lm.ldff, lm.d_moe_y, W, rows, c, st)));
+    const float* shared = L.shared_fused ? lm.d_moe_y + (size_t)M * k * W : nullptr;
+    if (s.shared_ff > 0 && !L.shared_fused) {
+        DenseCall g;
+        g.epi = kDenseGatedAct, g.act = s.act, g.n_out = s.shared_ff;
+        TM_PROF(P_GEMM_GATE_UP, TM_TRY(launch_dense_call(L.sh_gu, lm.d_h1, lm.ldw, lm.d_ff, lm.ldff, M, g, st)));
+        TM_PROF(P_GEMM_DOWN, TM_TRY(launch_dense_linear(L.sh_down, lm.d_ff, lm.ldff, lm.d_y2, W, M, kDenseScaleF32, 1.f, st)));
+        shared = lm.d_y2;
+    }
+    TM_PROF(P_GEMM_DOWN, TM_TRY(launch_moe_combine_f32(lm.d_y, lm.d_moe_y, lm.d_topk_w, lm.d_en2f, nullptr, 0, nullptr, M, W, k, true, st, true, shared,
+                                                 shared && s.shared_gate ? lm.d_proj + E : nullptr, lm.ldproj)));
+    return 0;
+}
+
+// one block with norms on both sides of its sublayers over M rows (see the head of this file); its normed input is ready.  `next`: the layer run
+// that follows (nullptr: none in this forward)
+static int both_layer(tm_engine* e, const LmLayer& L, const LmLayer* next, int M, const LmPart* parts, int nparts)
+{
+    LayeredModel&            lm = *e->lm;
+    const tm_layered_config& m  = lm.cfg;
+    const tm_layer_spec&     s  = L.spec;
+    hipStream_t              st = e->stream;
+    const int                W = m.width, H = s.heads;
+    if (s.mixer == TM_MIXER_RETENTION) {
+        TM_PROF(P_GEMM_QKV, TM_TRY(launch_dense_linear(L.qkv, lm.d_h1, lm.ldw, lm.d_proj, lm.ldproj, M, kDenseScaleF32, 1.f, st)));
+        for (int i = 0; i < nparts; ++i) {
+            const LmPart&  P  = parts[i];
+            StateMixParams sp = state_seqs(e, P);
+            sp.layer_offset   = L.state_offset;
+            sp.heads = H, sp.dim = s.dim, sp.vdim = s.vdim;
+            sp.proj = lm.d_proj + (size_t)P.row0 * lm.ldproj, sp.ld = lm.ldproj;
+            sp.c_q = 0, sp.c_k = L.c_k, sp.c_v = L.c_v;
+            sp.decay_h = L.decay_d;
+            sp.inv_freq = L.inv_freq, sp.rot_dims = s.rot_dims, sp.k_mult = (float)std::pow((double)s.dim, -0.5);
+            sp.rows = P.rows, sp.blocks = lm.d_blocks, sp.blocks_floats = lm.blocks_floats;
+            sp.out = lm.d_mixo + (size_t)P.row0 * lm.ldmix, sp.ldo = lm.ldmix;
+            TM_PROF(P_ATTN, TM_TRY(launch_state_mix(sp, kStateRetention, st)));
+        }
+        TM_PROF(P_ATTN, TM_TRY(launch_gated_group_norm(lm.d_cat, lm.ldcat, lm.elem, lm.d_mixo, lm.ldmix, nullptr, lm.d_proj + L.c_g, lm.ldproj, M, H, s.vdim,
+                                                       m.norm_eps, st, true)));
+    }
+    else {
+        DenseCall pc;
+        pc.epi = kDenseScaleF32, pc.n_seg = L.n_seg, pc.x_col_stride = lm.ldw;
+        std::copy(L.seg_n0, L.seg_n0 + L.n_seg, pc.seg_n0);
+        TM_PROF(P_GEMM_QKV, TM_TRY(launch_dense_call(L.qkv, lm.d_mix, lm.ldmixin, lm.d_proj, lm.ldproj, M, pc, st)));
+        // ---- left: windowed attention over convolved projections ----
+        for (int i = 0; i < nparts; ++i) {
+            const LmPart&     P = parts[i];
+            GeneralAttnParams p = attn_params(e, L, P);
+            AttnPrepExtra     ex;
+            ex.inv_freq = L.inv_freq, ex.rot_dims = s.rot_dims, ex.v_mult = s.left_scale;
+            const float* from = lm.d_proj + (size_t)P.row0 * lm.ldproj;
+            int          ldf  = lm.ldproj;
+            if (L.conv_taps > 0 && P.decode) {  // one row per sequence: the convolution runs inside the prepare kernel
+                ex.conv_w = L.conv_w, ex.conv_taps = L.conv_taps, ex.conv_ch = L.conv_ch;
+                ex.conv_state = lm.d_state, ex.conv_slot_stride = lm.state_slot_floats, ex.conv_offset = L.conv_offset;
+                ex.conv_slot0 = P.slot0, ex.conv_park_slot = e->cfg.max_batch_size, ex.conv_active = P.active;
+            }
+            else if (L.conv_taps > 0) {
+                StateMixParams sp = state_seqs(e, P);
+                sp.layer_offset   = L.conv_offset;
+                float* conv       = lm.d_conv + (size_t)P.row0 * lm.ldconv;
+                TM_PROF(P_KV_STORE, TM_TRY(launch_short_conv(conv, lm.ldconv, from, ldf, 0, L.conv_w, L.conv_ch, L.conv_taps, 0, sp, st)));
+                from = conv, ldf = lm.ldconv;
+            }
+            TM_PROF(P_KV_STORE, TM_TRY(launch_attn_prep(from, ldf, 0, L.c_k, L.c_v, (void*)p.q, lm.ldq, false, false, m.norm_eps, p, st, ex)));
+        }
+        TM_TRY(run_attention_parts(e, L, parts, nparts));
+        // ---- right: the time mixer ----
+        const int Hr = s.r_heads, dr = s.r_dim;
+        TM_PROF(P_KV_STORE, TM_TRY(launch_act_cast_f32(lm.d_lora, lm.ldlora, lm.elem, lm.d_proj + L.c_w1, lm.ldproj, M, s.decay_rank, 1, st)));
+        DenseCall c;
+        c.epi  = kDenseBiasF32;
+        c.bias = L.w0;
+        TM_PROF(P_GEMM_QKV, TM_TRY(launch_dense_call(L.w2, lm.d_lora, lm.ldlora, lm.d_wdec, lm.ldmix, M, c, st)));
+        for (int i = 0; i < nparts; ++i) {
+            const LmPart&  P  = parts[i];
+            StateMixParams sp = state_seqs(e, P);
+            sp.layer_offset   = L.state_offset;
+            sp.heads = Hr, sp.dim = dr, sp.vdim = dr;
+            sp.proj = lm.d_proj + (size_t)P.row0 * lm.ldproj, sp.ld = lm.ldproj;
+            sp.c_q = L.c_rr, sp.c_k = L.c_rk, sp.c_v = L.c_rv;
+            sp.decay_w = lm.d_wdec + (size_t)P.row0 * lm.ldmix, sp.ld_w = lm.ldmix;
+            sp.bonus = L.bonus;
+            sp.rows = P.rows, sp.blocks = lm.d_blocks, sp.blocks_floats = lm.blocks_floats;
+            sp.out = lm.d_mixo + (size_t)P.row0 * lm.ldmix, sp.ldo = lm.ldmix;
+            TM_PROF(P_ATTN, TM_TRY(launch_state_mix(sp, kStateBonus, st)));
+        }
+        TM_PROF(P_ATTN, TM_TRY(launch_gated_group_norm((char*)lm.d_cat + (size_t)L.n_att * lm.elem, lm.ldcat, lm.elem, lm.d_mixo, lm.ldmix, L.r_norm,
+                                                       lm.d_proj + L.c_rg, lm.ldproj, M, Hr, dr, m.norm_eps, st, true, s.right_scale)));
+    }
+    TM_PROF(P_GEMM_O, TM_TRY(launch_dense_linear(L.wo, lm.d_cat, lm.ldcat, lm.d_y, W, M, kDenseScaleF32, 1.f, st)));
+    const float* x0     = next && m.loop_add && next->spec.loop_pass > 0 ? lm.d_x0 : nullptr;
+    const float* next_w = next ? next->norm1 : nullptr;
+    if (s.mlp == TM_MLP_NONE) {
+        return close_block(e, lm.d_y, L.norm1b, x0, next_w, next, M, parts, nparts);
+    }
+    TM_TRY(close_block(e, lm.d_y, L.norm1b, nullptr, L.norm2, nullptr, M, parts, nparts));
+    if (s.mlp == TM_MLP_MOE) {
+        TM_TRY(grouped_experts(e, L, M));
+    }
+    else {
+        DenseCall c;  // the clamped pair leaves the [gate | up] product's epilogue in the activation type
+        c.epi   = kDenseGatedAct;
+        c.act   = s.act;
+        c.n_out = s.ff;
+        c.act_limit = s.act_limit, c.act_alpha = s.act_alpha;
+        TM_PROF(P_GEMM_GATE_UP, TM_TRY(launch_dense_call(L.gu, lm.d_h1, lm.ldw, lm.d_ff, lm.ldff, M, c, st)));
+        TM_PROF(P_GEMM_DOWN, TM_TRY(launch_dense_linear(L.down, lm.d_ff, lm.ldff, lm.d_y, W, M, kDenseScaleF32, 1.f, st)));
+    }
+    return close_block(e, lm.d_y, L.norm2b, x0, next_w, next, M, parts, nparts);
+}
+
 // the layer loop over M rows described by `parts`; leaves the residual stream in lm.d_res
 static int layered_layers(tm_engine* e, const int* d_ids, int M, const LmPart* parts, int nparts)
 {
@@ -1523,7 +1856,7 @@ static int layered_layers(tm_engine* e, const int* d_ids, int M, const LmPart* p
         TM_TRY(launch_rows_prepare(lm.d_row_seq + P.row0, lm.d_row_pos + P.row0, P.cu_q, P.k_len, P.nseq, P.rows, st));
     }
     TM_PROF(P_EMBED, TM_TRY(launch_embedding_f32(lm.d_res, lm.embed, lm.elem, d_ids, M, m.width, m.vocab, st, m.embed_scale != 0.f ? m.embed_scale : 1.f,
-                                                  lm.d_hist)));
+                                                  m.loop_add ? lm.d_x0 : lm.d_hist)));
     if (m.loop_times > 0) {  // the embedding output is read again where a loop pass begins
         TM_PROF(P_EMBED, TM_TRY(launch_embedding_f32(lm.d_x0, lm.embed, lm.elem, d_ids, M, m.width, m.vocab, st)));
     }
@@ -1531,12 +1864,19 @@ static int layered_layers(tm_engine* e, const int* d_ids, int M, const LmPart* p
     for (int li = 0; li < n_run; ++li) {
         const LmLayer&       L = lm.layers[li];
         const tm_layer_spec& s = L.spec;
-        if (s.loop_pass >= 0) {
+        if (s.loop_pass >= 0 && m.loop_times > 0) {
             DenseCall c;
             c.epi  = kDenseBiasF32;
             c.bias = lm.loop_step + (size_t)s.loop_pass * m.width;
             TM_PROF(P_RES_NORM, TM_TRY(launch_concat2(lm.d_xx, lm.ld2w, lm.elem, lm.d_res, lm.d_x0, M, m.width, st)));
             TM_PROF(P_GEMM_O, TM_TRY(launch_dense_call(lm.loop_in, lm.d_xx, lm.ld2w, lm.d_res, m.width, M, c, st)));
+        }
+        if (L.both) {
+            if (li == 0) {
+                TM_TRY(close_block(e, nullptr, nullptr, nullptr, L.norm1, &L, M, parts, nparts));
+            }
+            TM_TRY(both_layer(e, L, li + 1 < n_run ? &lm.layers[li + 1] : nullptr, M, parts, nparts));
+            continue;
         }
         if (L.pre) {
             if (li == 0) {
@@ -1640,6 +1980,51 @@ int layered_forward(tm_engine* e, const int* d_ids, int M, int nseq, bool decode
     return layered_head(e, e->d_rows, nseq, slot0, d_ids + nd, e->d_cu_q, M - nd, e->d_k_len, nullptr);  // d_rows: last row of every sequence
 }
 
+// what a block with norms on both sides of its sublayers may hold
+static int validate_both_layer(const tm_layered_config* m, int i)
+{
+    const tm_layer_spec& s  = m->layers[i];
+    const std::string    at = "layer " + std::to_string(i);
+    TM_REQUIRE(!m->final_layer_norm && m->norm_groups == 0 && m->loop_times == 0 && m->residual_mult == 1.f && m->side_dim == 0 && !m->depth_avg,
+               at + ": both_norms blocks end in an RMS norm, without loop tensors, residual multiplier, token-side input or depth average");
+    TM_REQUIRE(!s.post_norm && !s.pre_norm && !s.one_norm && !s.resid_gate && !s.dist_bias && !s.out_gate && s.chunk == 0 && !s.qk_unit_norm && !s.v_unit_norm
+                   && s.qtemp_coef == 0.f && !s.qkv_bias && !s.qk_norm_w && s.keep_first == 0 && s.norm_groups == 0 && !s.diff_maps && s.yarn_factor == 0.f
+                   && !s.rot_pairs && !s.expert_plain && !s.router_softmax,
+               at + ": a both_norms block takes none of the other block forms' switches");
+    TM_REQUIRE(s.heads >= 1 && s.kv_heads >= 1 && s.heads % s.kv_heads == 0 && s.dim >= 1 && s.dim <= 256 && s.vdim >= 1 && s.vdim <= 256,
+               at + ": heads % kv_heads, 1 <= dim, vdim <= 256");
+    TM_REQUIRE(s.rot_dims >= 0 && s.rot_dims % 2 == 0 && s.rot_dims <= s.dim && s.rot_base > 0.f && s.rot_scale > 0.f,
+               at + ": rot_dims even and <= dim, rot_base, rot_scale > 0");
+    if (s.mixer == TM_MIXER_RETENTION) {
+        TM_REQUIRE(s.kv_heads == s.heads && s.decay && s.window == 0 && s.conv_taps == 0 && !s.sink && s.softcap <= 0.f,
+                   at + ": retention: one decay and one key / value head per head, no window / convolution / sink / cap");
+    }
+    else {
+        TM_REQUIRE(s.mixer == TM_MIXER_PARALLEL, at + ": a both_norms block mixes by retention or by the parallel pair");
+        TM_REQUIRE(s.conv_taps >= 0 && s.conv_taps <= 16 && s.window >= 0, at + ": left mixer: at most 16 taps, window >= 0");
+        TM_REQUIRE(s.r_heads >= 1 && s.r_kv_heads == s.r_heads && s.r_dim >= 1 && s.r_dim <= 256 && s.r_vdim == s.r_dim && s.decay_rank >= 1,
+                   at + ": right mixer: r_kv_heads = r_heads, 1 <= r_dim = r_vdim <= 256, decay_rank >= 1");
+    }
+    TM_REQUIRE(s.mlp == TM_MLP_NONE || (s.mlp == TM_MLP_GATED && s.ff >= 1 && (s.act == TM_ACT_SILU || s.act == TM_ACT_GELU_TANH || s.act == TM_ACT_RELU2 || (s.act == TM_ACT_CLAMPED && s.act_limit >= 0.f)))
+                   || (s.mlp == TM_MLP_MOE && s.ff >= 1 && s.act >= TM_ACT_RELU2 && s.act <= TM_ACT_SILU && s.experts >= 1 && s.experts <= 1023 && s.shared_ff >= 0),
+               at + ": feed-forward of a both_norms block: gated (clamped | silu | gelu | relu^2) or gated experts");
+    if (s.mlp == TM_MLP_MOE) {
+        const int groups = std::max(1, s.group_count), keep = std::max(1, s.group_keep);
+        TM_REQUIRE(groups <= 256 && s.experts % groups == 0 && keep <= groups && s.top >= 1 && s.top <= s.experts / groups * keep,
+                   at + ": the groups divide the experts and the kept ones hold at least `top` of them");
+        TM_REQUIRE(!s.shared_gate || s.shared_ff > 0, at + ": shared_gate needs a shared expert");
+    }
+    TM_REQUIRE(s.weights_of < 0 || (s.weights_of < i && m->layers[s.weights_of].weights_of < 0), at + ": weights_of must name an earlier layer with tensors of its own");
+    if (s.weights_of >= 0) {
+        const tm_layer_spec& o = m->layers[s.weights_of];
+        TM_REQUIRE(o.mixer == s.mixer && o.heads == s.heads && o.kv_heads == s.kv_heads && o.dim == s.dim && o.vdim == s.vdim && o.mlp == s.mlp && o.ff == s.ff
+                       && o.experts == s.experts && o.top == s.top && o.conv_taps == s.conv_taps && o.r_heads == s.r_heads && o.r_dim == s.r_dim
+                       && o.decay_rank == s.decay_rank && o.shared_ff == s.shared_ff && o.rot_dims == s.rot_dims && o.sink == s.sink,
+                   at + ": form or sizes differ from the layer whose weights it uses");
+    }
+    return 0;
+}
+
 }  // namespace tmk
 
 extern "C" {
@@ -1658,7 +2043,17 @@ int tm_engine_create_layered(tm_engine** out, const tm_engine_config* c, const t
     for (int i = 0; i < m->n_layers; ++i) {
         const tm_layer_spec& s = m->layers[i];
         const std::string at = "layer " + std::to_string(i);
-        TM_REQUIRE(s.mixer >= TM_MIXER_ATTENTION && s.mixer <= TM_MIXER_FORGET, at + ": unknown mixer");
+        TM_REQUIRE(s.mixer >= TM_MIXER_ATTENTION && s.mixer <= TM_MIXER_RETENTION, at + ": unknown mixer");
+        TM_REQUIRE((s.both_norms != 0) == (m->layers[0].both_norms != 0), at + ": both_norms blocks do not mix with the other block forms");
+        if (s.both_norms) {
+            if (int rc = validate_both_layer(m, i)) {
+                return rc;
+            }
+            continue;
+        }
+        TM_REQUIRE(!m->loop_add && !m->tied_head && s.mixer != TM_MIXER_RETENTION && s.act != TM_ACT_CLAMPED && s.group_count == 0 && s.group_keep == 0
+                       && !s.router_correction && !s.router_renorm && !s.shared_gate,
+                   at + ": retention, the clamped activation, grouped routers, gated shared experts, tied heads and added loop inputs belong to both_norms blocks");
         TM_REQUIRE((s.pre_norm != 0) == (m->layers[0].pre_norm != 0), at + ": pre_norm blocks do not mix with the other block forms");
         if (s.pre_norm) {
             TM_REQUIRE(m->final_layer_norm && m->norm_groups == 0 && m->loop_times == 0 && m->residual_mult == 1.f, at + ": pre_norm blocks end in a final layer norm, without loop or residual multiplier");
@@ -1803,14 +2198,104 @@ int tm_engine_create_layered(tm_engine** out, const tm_engine_config* c, const t
         L.a_dim = L.spec.dim, L.a_vdim = L.spec.vdim, L.a_kv = L.spec.kv_heads, L.a_heads = L.spec.heads;
         L.post = L.spec.post_norm != 0;
         L.has_state = L.spec.mixer == TM_MIXER_LIGHTNING || L.spec.mixer == TM_MIXER_DELTA || L.spec.mixer == TM_MIXER_PARALLEL
-                      || L.spec.mixer == TM_MIXER_FORGET;
-        L.has_cache = L.spec.mixer != TM_MIXER_LIGHTNING && L.spec.mixer != TM_MIXER_DELTA && L.spec.mixer != TM_MIXER_FORGET;
+                      || L.spec.mixer == TM_MIXER_FORGET || L.spec.mixer == TM_MIXER_RETENTION;
+        L.has_cache = L.spec.mixer != TM_MIXER_LIGHTNING && L.spec.mixer != TM_MIXER_DELTA && L.spec.mixer != TM_MIXER_FORGET
+                      && L.spec.mixer != TM_MIXER_RETENTION;
+        L.both = L.spec.both_norms != 0;
         L.pre  = L.spec.pre_norm != 0;
-        L.wide = !L.post && !L.pre && layer_wide(L.spec);
+        L.wide = !L.post && !L.pre && !L.both && layer_wide(L.spec);
         auto slot = [&](const std::string& name, int64_t rows, int64_t cols) {
             e->slots[name].bytes = rows * cols * 2;
             lm.fan_in[name]      = (int)cols;
         };
+        if (L.both) {
+            const tm_layer_spec& s = L.spec;
+            lm.has_both = true;
+            L.c_k = L.n_q, L.c_v = L.c_k + L.n_k, L.c_g = L.c_end = L.c_v + L.n_v;
+            if (s.mixer == TM_MIXER_RETENTION) {
+                L.c_end = L.c_g + L.n_att;
+                L.decay_h.assign(s.decay, s.decay + s.heads);
+            }
+            else {
+                auto up128  = [](int n) { return (n + 127) / 128 * 128; };
+                L.r_nv      = s.r_heads * s.r_dim;
+                L.conv_ch   = L.c_end, L.conv_taps = s.conv_taps;
+                L.n_seg     = 6;
+                L.c_rr = up128(L.c_end), L.c_rk = up128(L.c_rr + L.r_nv), L.c_rv = up128(L.c_rk + L.r_nv), L.c_rg = up128(L.c_rv + L.r_nv);
+                L.c_w1 = up128(L.c_rg + L.r_nv), L.c_end = L.c_w1 + s.decay_rank;
+                const int seg[6] = {0, L.c_rr, L.c_rk, L.c_rv, L.c_rg, L.c_w1};
+                std::copy(seg, seg + 6, L.seg_n0);
+            }
+            L.spec.decay   = nullptr;  // (the caller's memory)
+            L.shared_fused = s.mlp == TM_MLP_MOE && s.shared_ff > 0 && s.shared_ff <= s.ff;
+            if (L.src != i) {
+                continue;
+            }
+            slot(lname(i, "norm1"), 1, W);
+            slot(lname(i, "norm1b"), 1, W);
+            if (s.mixer == TM_MIXER_RETENTION) {
+                slot(lname(i, "mix.q"), L.n_q, W);
+                slot(lname(i, "mix.k"), L.n_k, W);
+                slot(lname(i, "mix.v"), L.n_v, W);
+                slot(lname(i, "mix.g"), L.n_att, W);
+                slot(lname(i, "mix.o"), W, L.n_att);
+            }
+            else {
+                const int n_r = L.r_nv;
+                slot(lname(i, "mix.left.q"), L.n_q, W);
+                slot(lname(i, "mix.left.k"), L.n_k, W);
+                slot(lname(i, "mix.left.v"), L.n_v, W);
+                if (s.conv_taps > 0) {
+                    slot(lname(i, "mix.left.q.conv"), L.n_q, s.conv_taps);
+                    slot(lname(i, "mix.left.k.conv"), L.n_k, s.conv_taps);
+                    slot(lname(i, "mix.left.v.conv"), L.n_v, s.conv_taps);
+                }
+                if (s.sink) {
+                    slot(lname(i, "mix.left.sink"), 1, s.heads);
+                }
+                slot(lname(i, "mix.left.o"), W, L.n_att);
+                for (const char* t : {"r", "k", "v", "g", "w"}) {
+                    slot(lname(i, (std::string("mix.right.mu.") + t).c_str()), 1, W);
+                    if (*t != 'w') {
+                        slot(lname(i, (std::string("mix.right.") + t).c_str()), n_r, W);
+                    }
+                }
+                slot(lname(i, "mix.right.w1"), s.decay_rank, W);
+                slot(lname(i, "mix.right.w2"), n_r, s.decay_rank);
+                slot(lname(i, "mix.right.w0"), 1, n_r);
+                slot(lname(i, "mix.right.u"), 1, n_r);
+                slot(lname(i, "mix.right.norm"), 1, n_r);
+                slot(lname(i, "mix.right.o"), W, n_r);
+            }
+            auto gated = [&](const std::string& pre, int ff) {
+                slot(lname(i, (pre + "gate").c_str()), ff, W);
+                slot(lname(i, (pre + "up").c_str()), ff, W);
+                slot(lname(i, (pre + "down").c_str()), W, ff);
+            };
+            if (s.mlp) {
+                slot(lname(i, "norm2"), 1, W);
+                slot(lname(i, "norm2b"), 1, W);
+            }
+            if (s.mlp == TM_MLP_GATED) {
+                gated("mlp.", s.ff);
+            }
+            else if (s.mlp == TM_MLP_MOE) {
+                slot(lname(i, "mlp.router"), s.experts, W);
+                if (s.router_correction) {
+                    slot(lname(i, "mlp.correction"), 1, s.experts);
+                }
+                for (int x = 0; x < s.experts; ++x) {
+                    gated("mlp.e" + std::to_string(x) + ".", s.ff);
+                }
+                if (s.shared_ff > 0) {
+                    gated("mlp.shared.", s.shared_ff);
+                }
+                if (s.shared_gate) {
+                    slot(lname(i, "mlp.shared.sg"), 1, W);
+                }
+            }
+            continue;
+        }
         if (L.pre) {
             const tm_layer_spec& s = L.spec;
             const int            H = s.heads, C = s.kv_rank, R = s.rot_dim;
@@ -2107,7 +2592,9 @@ int tm_engine_create_layered(tm_engine** out, const tm_engine_config* c, const t
     if (m->final_layer_norm && m->norm_groups == 0) {
         e->slots["final.norm.b"].bytes = W * 2;
     }
-    e->slots["head"].bytes       = W * m->vocab * 2;
+    if (!m->tied_head) {
+        e->slots["head"].bytes = W * m->vocab * 2;
+    }
     *out = e;
     return 0;
 }

@@ -21,6 +21,8 @@
 // A launch may be BATCHED (DenseCall::count > 1, grid z): item g multiplies with image g of the weight (images at a fixed stride), reads
 // x at column g * x_col_stride and writes y at column g * y_col_stride -- per-head projections of one activation row -- or, with
 // row_offsets, owns the rows [row_offsets[g], row_offsets[g + 1]) of x and y: the experts of a mixture over rows sorted by expert.
+// A launch may also have SEGMENTS (DenseCall::n_seg): ranges of output columns that read x at columns of their own -- the projections of
+// several inputs derived from one token (each its own mix of the token and its predecessor) as one product of any widths.
 #include "tm_kernels.h"
 
 namespace tmk {
@@ -68,14 +70,29 @@ __device__ __forceinline__ void dense_epilogue(void* y, int ldy, int m, int n, f
     }
 }
 
+// gate / up pair of a gated feed-forward
+__device__ __forceinline__ float dense_gated(const DenseCall& c, float g, float u)
+{
+    if (c.act == kActClamped) {
+        g = fminf(g, c.act_limit);
+        u = fminf(fmaxf(u, -c.act_limit), c.act_limit);
+        return g / (1.f + expf(-c.act_alpha * g)) * (u + 1.f);
+    }
+    return act_apply(c.act, g) * u;
+}
+
 // the item of a batched launch: where its operands start, and its row count (<= 0: nothing to do)
 struct DenseItem {
     size_t x_off, w_off;
     int    row_base, col_base, M;
 };
-__device__ __forceinline__ DenseItem dense_item(const DenseCall& c, int g, int M, int ldx)
+__device__ __forceinline__ DenseItem dense_item(const DenseCall& c, int g, int M, int ldx, int n0)
 {
     DenseItem it{(size_t)g * c.x_col_stride, (size_t)g * c.w_stride, 0, g * c.y_col_stride, M};
+#pragma unroll
+    for (int s = 1; s < kDenseMaxSeg; ++s) {  // (the segment of this workgroup's columns)
+        it.x_off += s < c.n_seg && n0 >= c.seg_n0[s] ? c.x_col_stride : 0;
+    }
     if (c.row_offsets) {
         it.row_base = c.row_offsets[g];
         it.x_off += (size_t)it.row_base * ldx;
@@ -97,7 +114,7 @@ __global__ __launch_bounds__(WAVES * 64) void dense_skinny_bf16_kernel(const __b
                                                                 void* __restrict__ y, int ldy, int M, int N, DenseCall call)
 {
     __shared__ float red[WAVES][MT * NT][64][4];
-    const DenseItem it = dense_item(call, blockIdx.y, M, ldx);
+    const DenseItem it = dense_item(call, blockIdx.y, M, ldx, blockIdx.x * 16 * NT);
     const int       row_base = it.row_base, col_base = it.col_base;
     M = it.M, x += it.x_off, w += it.w_off;
     if (M <= 0) {
@@ -205,7 +222,7 @@ __global__ __launch_bounds__(WAVES * 64) void dense_skinny_bf16_kernel(const __b
                 }
                 const int m = t * 16 + (l >> 4) * 4 + i, n = (n0 >> 1) + (l & 15);
                 if (m < M && n < call.n_out) {
-                    ((__bf16*)y)[(size_t)(row_base + m) * ldy + col_base + n] = (__bf16)(act_apply(call.act, g) * u);
+                    ((__bf16*)y)[(size_t)(row_base + m) * ldy + col_base + n] = (__bf16)dense_gated(call, g, u);
                 }
             }
         }
@@ -239,7 +256,7 @@ __global__ __launch_bounds__(256) void dense_tiled_bf16_kernel(const __bf16* __r
     __shared__ __attribute__((aligned(16))) __bf16 sb[2][kTN * kLdsRow];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const int m0 = blockIdx.y * TM, n0 = blockIdx.x * kTN;
-    const DenseItem it = dense_item(call, blockIdx.z, M, ldx);
+    const DenseItem it = dense_item(call, blockIdx.z, M, ldx, n0);
     const int       row_base = it.row_base, col_base = it.col_base;
     M = it.M, x += it.x_off, w += it.w_off;
     if (m0 >= M) {  // the whole workgroup: an item with fewer rows than the launch's largest
@@ -327,7 +344,7 @@ __global__ __launch_bounds__(256) void dense_tiled_bf16_kernel(const __bf16* __r
                 for (int q = 0; q < 4; ++q) {
                     const int m = m0 + wm + i * 16 + (lane >> 4) * 4 + q, n = ((n0 + wn) >> 1) + (j >> 1) * 16 + (lane & 15);
                     if (m < M && n < call.n_out) {
-                        ((__bf16*)y)[(size_t)(row_base + m) * ldy + col_base + n] = (__bf16)(act_apply(call.act, acc[i][j][q]) * acc[i][j + 1][q]);
+                        ((__bf16*)y)[(size_t)(row_base + m) * ldy + col_base + n] = (__bf16)dense_gated(call, acc[i][j][q], acc[i][j + 1][q]);
                     }
                 }
             }
@@ -360,7 +377,7 @@ __global__ __launch_bounds__(256) void dense_f32_kernel(const float* __restrict_
     __shared__ __attribute__((aligned(16))) float sb[16][64 + 4];
     const int tid = threadIdx.x;
     const int m0 = blockIdx.y * 64, n0 = blockIdx.x * 64;
-    const DenseItem it = dense_item(call, blockIdx.z, M, ldx);
+    const DenseItem it = dense_item(call, blockIdx.z, M, ldx, n0);
     const int       row_base = it.row_base, col_base = it.col_base;
     M = it.M, x += it.x_off, w += it.w_off;
     if (m0 >= M) {
@@ -402,7 +419,7 @@ __global__ __launch_bounds__(256) void dense_f32_kernel(const float* __restrict_
             for (int j = 0; j < 2; ++j) {
                 const int m = m0 + tr + i, n = ((n0 + tc) >> 1) + j;
                 if (m < M && n < call.n_out) {
-                    ((float*)y)[(size_t)(row_base + m) * ldy + col_base + n] = act_apply(call.act, acc[i][j]) * acc[i][j + 2];
+                    ((float*)y)[(size_t)(row_base + m) * ldy + col_base + n] = dense_gated(call, acc[i][j], acc[i][j + 2]);
                 }
             }
         }
@@ -531,6 +548,12 @@ int launch_dense_call(const DenseWeight& d, const void* x, int ldx, void* y, int
                                          && call.table_col + d.N <= call.ld_table),
                "dense linear: table");
     TM_REQUIRE(epi != kDenseResidGate || (call.gate && call.gate_bias && call.ldg >= d.N), "dense linear: gate");
+    TM_REQUIRE(call.n_seg >= 0 && call.n_seg <= kDenseMaxSeg && (call.n_seg == 0 || (call.count == 1 && call.seg_n0[0] == 0 && ldx >= d.Kp + (call.n_seg - 1) * call.x_col_stride)),
+               "dense linear: segments");
+    for (int s = 1; s < call.n_seg; ++s) {
+        TM_REQUIRE(call.seg_n0[s] % kTN == 0 && call.seg_n0[s] > call.seg_n0[s - 1] && call.seg_n0[s] < d.N, "dense linear: segment borders");
+    }
+    TM_REQUIRE(call.act != kActClamped || epi == kDenseGatedAct, "dense linear: the clamped activation takes a gate / up pair");
     if (M == 0) {
         return 0;
     }

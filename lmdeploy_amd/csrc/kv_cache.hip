@@ -486,7 +486,7 @@ __global__ __launch_bounds__(256) void attn_prep_kernel(const float* __restrict_
     else {
         T* v = (T*)(base + p.v_offset) + (size_t)head * n * p.block_len + ti;
         for (int i = lane; i < n; i += 64) {
-            v[(size_t)i * p.block_len] = (T)(x[i] * inv);
+            v[(size_t)i * p.block_len] = (T)(x[i] * (inv * ex.v_mult));
         }
     }
 }

@@ -424,12 +424,134 @@ int launch_moe_topk_softmax(int* ids, float* w, const float* logits, int ld, int
     return 0;
 }
 
+// Grouped router, one wave per token (four tokens per workgroup): the choice scores of a token lie in LDS, the lanes share the searches.
+constexpr int kGroupedMaxExperts = 1024, kGroupedMaxGroups = 256;
+
+__device__ __forceinline__ void wave_argmax(float& v, int& i)  // the largest v, the lower index on a tie (i = INT_MAX: no candidate)
+{
+#pragma unroll
+    for (int d = 1; d < 64; d <<= 1) {
+        const float ov = __shfl_xor(v, d);
+        const int   oi = __shfl_xor(i, d);
+        if (oi != 0x7fffffff && (i == 0x7fffffff || ov > v || (ov == v && oi < i))) {
+            v = ov, i = oi;
+        }
+    }
+}
+
+__global__ __launch_bounds__(256) void moe_topk_grouped_kernel(int* __restrict__ ids, float* __restrict__ w, const float* __restrict__ logits, int ld,
+                                                               const float* __restrict__ corr, int T, int E, int groups, int keep, int k, int renorm)
+{
+    extern __shared__ float lds_topk[];
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, t = blockIdx.x * 4 + wave;
+    float*    choice = lds_topk + (size_t)wave * (2 * E + groups);  // [E], choice score; then the group's place in the order below
+    float*    score  = choice + E;                                   // [E]
+    float*    gsum   = score + E;                                    // [groups]
+    const bool on = t < T;
+    if (on) {
+        for (int e = lane; e < E; e += 64) {
+            const float s = 1.f / (1.f + expf(-logits[(size_t)t * ld + e]));
+            score[e]  = s;
+            choice[e] = s + (corr ? corr[e] : 0.f);
+        }
+    }
+    __syncthreads();
+    const int per = E / groups;
+    if (on && keep < groups) {
+        for (int g = lane; g < groups; g += 64) {
+            float a = -INFINITY, b = -INFINITY;  // the group's two best
+            for (int e = g * per; e < (g + 1) * per; ++e) {
+                const float c = choice[e];
+                if (c > a) {
+                    b = a, a = c;
+                }
+                else if (c > b) {
+                    b = c;
+                }
+            }
+            gsum[g] = per > 1 ? a + b : a;
+        }
+    }
+    __syncthreads();
+    if (on && keep < groups) {
+        // group g stays if fewer than `keep` groups come before it; the others' experts leave the competition
+        for (int g = lane; g < groups; g += 64) {
+            int before = 0;
+            for (int o = 0; o < groups; ++o) {
+                before += gsum[o] > gsum[g] || (gsum[o] == gsum[g] && o < g);
+            }
+            if (before >= keep) {
+                for (int e = g * per; e < (g + 1) * per; ++e) {
+                    choice[e] = -INFINITY;
+                }
+            }
+        }
+    }
+    __syncthreads();
+    float sum = 0.f;
+    for (int j = 0; j < k; ++j) {
+        float v = -INFINITY;
+        int   i = 0x7fffffff;
+        if (on) {
+            for (int e = lane; e < E; e += 64) {
+                if (choice[e] > v) {
+                    v = choice[e], i = e;
+                }
+            }
+        }
+        wave_argmax(v, i);
+        i = min(i, E - 1);  // (the kept groups hold at least k experts: there is always a candidate)
+        if (on) {
+            const float s = score[i];
+            sum += s;
+            if (lane == 0) {
+                ids[(size_t)t * k + j] = i;
+                w[(size_t)t * k + j]   = s;
+                choice[i]              = -INFINITY;
+            }
+        }
+        __syncthreads();
+    }
+    if (on && renorm) {
+        const float inv = 1.f / (sum + 1e-20f);
+        for (int j = lane; j < k; j += 64) {
+            w[(size_t)t * k + j] *= inv;  // (written by lane 0 of this wave, ahead of the barrier above)
+        }
+    }
+}
+
+int launch_moe_topk_grouped(int* ids, float* w, const float* logits, int ld, const float* correction, int T, int E, int groups, int keep, int k,
+                            bool renorm, hipStream_t st)
+{
+    TM_REQUIRE(ids && w && logits && E >= 1 && E <= kGroupedMaxExperts && ld >= E, "moe grouped top-k: operands");
+    TM_REQUIRE(groups >= 1 && groups <= kGroupedMaxGroups && E % groups == 0 && keep >= 1 && keep <= groups && k >= 1 && k <= E / groups * keep,
+               "moe grouped top-k: the kept groups hold at least k experts");
+    if (T == 0) {
+        return 0;
+    }
+    const size_t lds = (size_t)4 * (2 * E + groups) * sizeof(float);
+    moe_topk_grouped_kernel<<<(T + 3) / 4, 256, lds, st>>>(ids, w, logits, ld, correction, T, E, groups, keep, k, renorm);
+    TM_HIP_CHECK(hipGetLastError());
+    return 0;
+}
+
 // rows sorted by expert: xs[en2f[j][t]] = (scale ? w[t][j] : 1) * x[t] -- the weight on the expert's INPUT
 template<class T>
 __global__ __launch_bounds__(256) void moe_gather_kernel(T* __restrict__ xs, int lds, const T* __restrict__ x, int ldx, const float* __restrict__ w,
-                                                         const int* __restrict__ en2f, int Tn, int H, int k, int scale)
+                                                         const int* __restrict__ en2f, int Tn, int H, int k, int scale, int* __restrict__ shared_offsets,
+                                                         int E)
 {
-    const int t = blockIdx.x / k, j = blockIdx.x % k;
+    const int kk = k + (shared_offsets ? 1 : 0);
+    const int t = blockIdx.x / kk, j = blockIdx.x % kk;
+    if (j == k) {  // the copy behind the routed rows
+        if (t == 0 && threadIdx.x == 0) {
+            shared_offsets[E + 1] = Tn * kk;
+        }
+        for (int i = threadIdx.x; i < H; i += 256) {
+            xs[((size_t)Tn * k + t) * lds + i] = x[(size_t)t * ldx + i];
+        }
+        return;
+    }
     const int f = en2f[(size_t)j * Tn + t];
     const float a = scale ? w[(size_t)t * k + j] : 1.f;
     for (int i = threadIdx.x; i < H; i += 256) {
@@ -438,17 +560,18 @@ __global__ __launch_bounds__(256) void moe_gather_kernel(T* __restrict__ xs, int
 }
 
 int launch_moe_gather(void* xs, int lds, const void* x, int ldx, int elem_bytes, const float* w, const int* en2f, int T, int H, int k, bool scale,
-                      hipStream_t st)
+                      hipStream_t st, int* shared_offsets, int E)
 {
     TM_REQUIRE(xs && x && w && en2f && lds >= H && ldx >= H, "moe gather: operands");
     if (T == 0) {
         return 0;
     }
+    const int wgs = T * (k + (shared_offsets ? 1 : 0));
     if (elem_bytes == 2) {
-        moe_gather_kernel<__bf16><<<T * k, 256, 0, st>>>((__bf16*)xs, lds, (const __bf16*)x, ldx, w, en2f, T, H, k, scale);
+        moe_gather_kernel<__bf16><<<wgs, 256, 0, st>>>((__bf16*)xs, lds, (const __bf16*)x, ldx, w, en2f, T, H, k, scale, shared_offsets, E);
     }
     else {
-        moe_gather_kernel<float><<<T * k, 256, 0, st>>>((float*)xs, lds, (const float*)x, ldx, w, en2f, T, H, k, scale);
+        moe_gather_kernel<float><<<wgs, 256, 0, st>>>((float*)xs, lds, (const float*)x, ldx, w, en2f, T, H, k, scale, shared_offsets, E);
     }
     TM_HIP_CHECK(hipGetLastError());
     return 0;
@@ -457,7 +580,7 @@ int launch_moe_gather(void* xs, int lds, const void* x, int ldx, int elem_bytes,
 // resid[t] += gate(t) * sum_j (weighted ? w[t][j] : 1) * y[en2f[j][t]], gate(t)[i] = sigmoid(gate[t][i] + gate_bias[i]) (gate == nullptr: 1)
 __global__ void moe_combine_f32_kernel(float* __restrict__ resid, const float* __restrict__ y, const float* __restrict__ w, const int* __restrict__ en2f,
                                        const float* __restrict__ gate, int ldg, const float* __restrict__ gate_bias, int Tn, int H, int k, int weighted,
-                                       int overwrite, const float* __restrict__ add)
+                                       int overwrite, const float* __restrict__ add, const float* __restrict__ add_gate, int ld_ag)
 {
     const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
     if (i >= (size_t)Tn * H) {
@@ -472,18 +595,21 @@ __global__ void moe_combine_f32_kernel(float* __restrict__ resid, const float* _
     if (gate) {
         s = s / (1.f + expf(-(gate[(size_t)t * ldg + c] + gate_bias[c])));
     }
-    resid[i] = overwrite ? (add ? add[i] + s : s) : resid[i] + s;
+    if (add) {
+        s = (add_gate ? add[i] / (1.f + expf(-add_gate[(size_t)t * ld_ag])) : add[i]) + s;
+    }
+    resid[i] = overwrite ? s : resid[i] + s;
 }
 
 int launch_moe_combine_f32(float* resid, const float* y, const float* w, const int* en2f, const float* gate, int ldg, const float* gate_bias, int T,
-                           int H, int k, bool weighted, hipStream_t st, bool overwrite, const float* add)
+                           int H, int k, bool weighted, hipStream_t st, bool overwrite, const float* add, const float* add_gate, int ld_add_gate)
 {
-    TM_REQUIRE(resid && y && w && en2f && (!gate || (gate_bias && ldg >= H)), "moe combine: operands");
+    TM_REQUIRE(resid && y && w && en2f && (!gate || (gate_bias && ldg >= H)) && (!add || overwrite) && (!add_gate || add), "moe combine: operands");
     const size_t total = (size_t)T * H;
     if (total == 0) {
         return 0;
     }
-    moe_combine_f32_kernel<<<(total + 255) / 256, 256, 0, st>>>(resid, y, w, en2f, gate, ldg, gate_bias, T, H, k, weighted, overwrite, add);
+    moe_combine_f32_kernel<<<(total + 255) / 256, 256, 0, st>>>(resid, y, w, en2f, gate, ldg, gate_bias, T, H, k, weighted, overwrite, add, add_gate, ld_add_gate);
     TM_HIP_CHECK(hipGetLastError());
     return 0;
 }

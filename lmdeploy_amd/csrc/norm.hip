@@ -524,6 +524,229 @@ int launch_layer_close(const LayerClose& c, hipStream_t st)
     return 0;
 }
 
+// one row between two RMS norms (see BlockClose); the row stays in registers (H <= NT * NR)
+template<class T, int NT, int NR>
+__global__ __launch_bounds__(NT) void block_close_kernel(BlockClose c)
+{
+    __shared__ float red[NT / 64];
+    const int    m = blockIdx.x, H = c.H;
+    const size_t r0 = (size_t)m * H;
+    float        v[NR];
+#pragma unroll
+    for (int q = 0; q < NR; ++q) {
+        const int i = threadIdx.x + q * NT;
+        v[q]        = i < H ? c.x[r0 + i] : 0.f;
+    }
+    if (c.y) {
+        float y[NR], ss = 0.f;
+#pragma unroll
+        for (int q = 0; q < NR; ++q) {
+            const int i = threadIdx.x + q * NT;
+            y[q]        = i < H ? c.y[r0 + i] : 0.f;
+            ss          = fmaf(y[q], y[q], ss);
+        }
+        const float inv = 1.0f / sqrtf(block_sum<NT>(ss, red) / (float)H + c.eps);
+#pragma unroll
+        for (int q = 0; q < NR; ++q) {
+            const int i = threadIdx.x + q * NT;
+            if (i < H) {
+                v[q] = fmaf(y[q] * inv, c.w_offset + c.post_w[i], v[q]);
+            }
+        }
+    }
+    float ss = 0.f;
+#pragma unroll
+    for (int q = 0; q < NR; ++q) {
+        const int i = threadIdx.x + q * NT;
+        if (c.x0 && i < H) {
+            v[q] += c.x0[r0 + i];
+        }
+        if ((c.y || c.x0) && i < H) {
+            c.x[r0 + i] = v[q];
+        }
+        ss = fmaf(v[q], v[q], ss);
+    }
+    if (!c.next_w) {
+        return;
+    }
+    const float inv = 1.0f / sqrtf(block_sum<NT>(ss, red) / (float)H + c.eps);
+#pragma unroll
+    for (int q = 0; q < NR; ++q) {
+        const int i = threadIdx.x + q * NT;
+        if (i < H) {
+            v[q] = v[q] * inv * (c.w_offset + c.next_w[i]);
+            ((T*)c.h)[(size_t)m * c.ldh + i] = (T)v[q];
+        }
+    }
+    if (m >= c.shift_rows) {
+        if (c.hf) {
+#pragma unroll
+            for (int q = 0; q < NR; ++q) {
+                const int i = threadIdx.x + q * NT;
+                if (i < H) {
+                    c.hf[r0 + i] = v[q];
+                }
+            }
+        }
+        return;
+    }
+    const StateMixParams& s    = c.shift.seqs;
+    int                   slot = s.seq_slot ? s.seq_slot[m] : s.slot0 + m;
+    if (s.active && !s.active[m]) {
+        slot = s.park_slot;
+    }
+    float*     state = s.state + (size_t)slot * s.slot_stride + s.layer_offset;
+    const bool first = s.k_len[m] <= 1;
+#pragma unroll
+    for (int q = 0; q < NR; ++q) {
+        const int i = threadIdx.x + q * NT;
+        if (i < H) {
+            const float d = (first ? 0.f : state[i]) - v[q];
+            T*          o = (T*)c.shift.out + (size_t)m * c.shift.ld + i;
+            for (int j = 0; j < c.shift.n_mix; ++j) {
+                o[(size_t)(1 + j) * c.shift.mix_stride] = (T)fmaf(d, c.shift.mu[(size_t)j * H + i], v[q]);
+            }
+            state[i] = v[q];
+        }
+    }
+}
+
+template<class T>
+static void launch_block_close_t(const BlockClose& c, hipStream_t st)
+{
+    if (c.M <= 256 && c.H > 1024 && c.H <= 8192) {  // few rows: latency counts, every wave the row can fill
+        if (c.H <= 4096) {
+            block_close_kernel<T, 1024, 4><<<c.M, 1024, 0, st>>>(c);
+        }
+        else {
+            block_close_kernel<T, 1024, 8><<<c.M, 1024, 0, st>>>(c);
+        }
+    }
+    else if (c.H <= 1024) {
+        block_close_kernel<T, 256, 4><<<c.M, 256, 0, st>>>(c);
+    }
+    else if (c.H <= 4096) {
+        block_close_kernel<T, 256, 16><<<c.M, 256, 0, st>>>(c);
+    }
+    else if (c.H <= 8192) {
+        block_close_kernel<T, 1024, 8><<<c.M, 1024, 0, st>>>(c);
+    }
+    else {
+        block_close_kernel<T, 1024, 32><<<c.M, 1024, 0, st>>>(c);
+    }
+}
+
+static bool token_shift_ok(const TokenShift& s, int H)
+{
+    return s.n_mix >= 1 && s.mu && s.out && s.mix_stride >= H && s.ld >= (s.n_mix + 1) * s.mix_stride && s.seqs.cu_q && s.seqs.k_len && s.seqs.state;
+}
+
+int launch_block_close(const BlockClose& c, hipStream_t st)
+{
+    TM_REQUIRE(c.x && c.M >= 0 && c.H >= 1 && c.H <= 32768 && (!c.y || c.post_w), "block_close: operands, width <= 32768");
+    TM_REQUIRE(!c.next_w || (c.h && c.ldh >= c.H && (c.h_elem_bytes == 2 || c.h_elem_bytes == 4)), "block_close: norm");
+    TM_REQUIRE(c.shift_rows >= 0 && c.shift_rows <= c.M
+                   && (c.shift_rows == 0 || (c.next_w && token_shift_ok(c.shift, c.H) && c.shift.elem_bytes == c.h_elem_bytes && c.shift.seqs.nseq == c.shift_rows)),
+               "block_close: token mixes");
+    if (c.M == 0) {
+        return 0;
+    }
+    if (c.h_elem_bytes == 2) {
+        launch_block_close_t<__bf16>(c, st);
+    }
+    else {
+        launch_block_close_t<float>(c, st);
+    }
+    TM_HIP_CHECK(hipGetLastError());
+    return 0;
+}
+
+// token mixes of prompt portions, one workgroup per row, VEC channels per thread.  The workgroup of a sequence's first row -- the only one that
+// reads the state -- then stores its new content, the sequence's last row.
+template<class T, int VEC>
+__global__ __launch_bounds__(256) void token_shift_kernel(const float* __restrict__ h, TokenShift c, const int* __restrict__ row_seq,
+                                                          const int* __restrict__ row_pos, int H)
+{
+    typedef float VF __attribute__((ext_vector_type(VEC)));
+    typedef T     VT __attribute__((ext_vector_type(VEC)));
+    const StateMixParams& p = c.seqs;
+    const int   t = blockIdx.x, s = row_seq[t], row0 = p.cu_q[s] - p.cu_q[0];
+    const bool  first = t == row0, zero = first && row_pos[t] <= 0;
+    int         slot = p.seq_slot ? p.seq_slot[s] : p.slot0 + s;
+    if (p.active && !p.active[s]) {
+        slot = p.park_slot;
+    }
+    float*       state = p.state + (size_t)slot * p.slot_stride + p.layer_offset;
+    const float* prev  = first ? state : h + (size_t)(t - 1) * H;
+    const float* last  = h + (size_t)(p.cu_q[s + 1] - p.cu_q[0] - 1) * H;
+    auto load = [](const float* a) {
+        VF v;
+        if constexpr (VEC == 1) {
+            v[0] = a[0];
+        }
+        else {
+#pragma unroll
+            for (int e = 0; e < VEC; e += 4) {
+                const floatx4 u = *(const floatx4*)(a + e);
+#pragma unroll
+                for (int j = 0; j < 4; ++j) {
+                    v[e + j] = u[j];
+                }
+            }
+        }
+        return v;
+    };
+    for (int i = threadIdx.x * VEC; i < H; i += 256 * VEC) {
+        const VF v = load(h + (size_t)t * H + i);
+        VF       d = load(prev + i);  // (state rows start at a multiple of four floats)
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) {
+            d[e] = (zero ? 0.f : d[e]) - v[e];
+        }
+        T* o = (T*)c.out + (size_t)t * c.ld + i;
+        for (int j = 0; j < c.n_mix; ++j) {
+            const VF mu = load(c.mu + (size_t)j * H + i);
+            VT       y;
+#pragma unroll
+            for (int e = 0; e < VEC; ++e) {
+                y[e] = (T)fmaf(d[e], mu[e], v[e]);
+            }
+            *(VT*)(o + (size_t)(1 + j) * c.mix_stride) = y;
+        }
+        if (first) {
+#pragma unroll
+            for (int e = 0; e < VEC; ++e) {
+                state[i + e] = last[i + e];
+            }
+        }
+    }
+}
+
+int launch_token_shift(const float* h, const TokenShift& s, const int* row_seq, const int* row_pos, int rows, int H, hipStream_t st)
+{
+    TM_REQUIRE(h && row_seq && row_pos && H >= 1 && token_shift_ok(s, H) && (s.elem_bytes == 2 || s.elem_bytes == 4), "token_shift: operands");
+    if (rows == 0) {
+        return 0;
+    }
+    const bool vec = H % 8 == 0 && s.ld % 8 == 0 && s.mix_stride % 8 == 0 && s.seqs.slot_stride % 4 == 0 && s.seqs.layer_offset % 4 == 0;
+    if (s.elem_bytes == 2) {
+        if (vec) {
+            token_shift_kernel<__bf16, 8><<<rows, 256, 0, st>>>(h, s, row_seq, row_pos, H);
+        }
+        else {
+            token_shift_kernel<__bf16, 1><<<rows, 256, 0, st>>>(h, s, row_seq, row_pos, H);
+        }
+    }
+    else if (vec) {
+        token_shift_kernel<float, 8><<<rows, 256, 0, st>>>(h, s, row_seq, row_pos, H);
+    }
+    else {
+        token_shift_kernel<float, 1><<<rows, 256, 0, st>>>(h, s, row_seq, row_pos, H);
+    }
+    TM_HIP_CHECK(hipGetLastError());
+    return 0;
+}
+
 // PolyNorm: three statistics of a row (mean squares of z, z^2, z^3), then a cubic per element with the statistics folded into its coefficients.
 // The row stays in registers (n <= NT * NR) or is read twice (NR = 0)
 template<class T, int NT, int NR>

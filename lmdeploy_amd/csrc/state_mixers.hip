@@ -7,6 +7,9 @@
 //                                    w = g, u = g k, a u = beta k and the key beta k (launch_gdelta_prep forms these vectors)
 //   forget-gate linear attention:    S <- diag(f) S + (1 - f) v^T                      o = S^T q      q = silu(projection), f per key channel,
 //                                    f = low + (1 - low) sigmoid(logit + bias)
+//   retention:                       S <- decay[head] S + k v^T                         o = S^T q      q, k rotated by position, k scaled
+//   bonus recurrence:                o = (S + diag(u) k v^T)^T q;  S <- diag(w) S + k v^T            w = exp(-exp(logit)) per key channel; the
+//                                    current token enters o through the bonus u only
 //   short convolution:               y_t = sum_j w[:, j] u_(t - taps + 1 + j) per channel; its state is the last taps - 1 inputs
 //
 // State pool: one state per (slot, layer run) -- slot = the engine's batch slot of the sequence, plus one parking slot for the decode
@@ -25,7 +28,8 @@
 // stage of T <= TB tokens at once, which replaces T dependent steps by independent sums:
 //   o_t = decay^(t+1) S0^T q_t + sum_{j <= t} decay^(t-j) (q_t . k_j) v_j          S_T = decay^T S0 + sum_j decay^(T-1-j) k_j v_j^T
 // -- the pair products (q_t . k_j) decay^(t-j) are formed once per workgroup (one thread per pair) and shared by all columns.
-// The forget-gate mixer takes this kernel for decoded tokens; its prompt portions run in chunks on the matrix cores (below).
+// The forget-gate mixer, retention and the bonus recurrence take this kernel for decoded tokens; their prompt portions run in chunks on the
+// matrix cores (below).
 // One kernel serves prompt portions (many rows per sequence) and decoded tokens (one row, TB = 1): the state traffic of a decode step,
 // 2 * dim * vdim * 4 bytes per head, is what bounds it.
 #include "tm_kernels.h"
@@ -40,21 +44,47 @@ __device__ __forceinline__ float sm_silu(float z)
     return z / (1.f + expf(-z));
 }
 
+// staged vectors per token: q, k; the delta rule's decays, a u and u; the forget gates; the bonus recurrence's decays and u k
+__host__ __device__ constexpr int state_vectors(int kind)
+{
+    return kind == kStateDelta ? 5 : kind == kStateBonus ? 4 : kind == kStateForget ? 3 : 2;
+}
+
+// channel d of a query / key head turned to position pos (first rot_dims channels; channel i pairs with i + rot_dims / 2), fp32
+struct Rotation {
+    float sn = 0.f, cs = 1.f;
+    int   partner = 0;
+    __device__ __forceinline__ Rotation(const StateMixParams& p, int pos, int d)
+    {
+        const int half = p.rot_dims >> 1;
+        if (d < p.rot_dims) {
+            sincosf((float)pos * p.inv_freq[d < half ? d : d - half], &sn, &cs);
+            partner = d < half ? half : -half;
+            sn      = d < half ? -sn : sn;
+        }
+    }
+    __device__ __forceinline__ float operator()(const float* x) const  // x: the channel itself
+    {
+        return x[0] * cs + x[partner] * sn;
+    }
+};
+
 size_t state_mix_floats(int heads, int dim, int vdim)
 {
     const int wcols = kStateCW * kStateNC;
     return (size_t)heads * ((vdim + wcols - 1) / wcols) * ((dim + 7) / 8) * 64 * kStateNC;
 }
 
-// grid (nseq, heads, ceil(vdim / 64)), 256 threads, dynamic LDS = 2 * tb * (NV * dim + 64) floats (+ TB * TB for linear attention); NV = 2 | 3 | 5
+// grid (nseq, heads, ceil(vdim / 64)), 256 threads, dynamic LDS = 2 * tb * (NV * dim + 64) floats (+ TB * TB for linear attention); NV = 2 ... 5
 // staged vectors per token, tb = min(TB, max_q_len) tokens per stage, TB: as many as keep the buffers under 64 KB.
 // EXACT: dim == 8 * DQ -- every LDS stride is a compile-time constant and the per-token vectors are read 16 bytes at a time
 template<int DQ, int KIND, int TB, bool EXACT>
 __global__ __launch_bounds__(256) void state_mix_kernel(StateMixParams p)
 {
     extern __shared__ __attribute__((aligned(16))) float lds_all[];
-    constexpr bool DELTA = KIND == kStateDelta, LINEAR = KIND == kStateLinear, FORGET = KIND == kStateForget;
-    constexpr int NV = DELTA ? 5 : FORGET ? 3 : 2, CW = kStateCW, NC = kStateNC, RG = 64 / CW, WV = CW * NC, WC = 4 * WV;
+    constexpr bool DELTA = KIND == kStateDelta, LINEAR = KIND == kStateLinear, FORGET = KIND == kStateForget, RETAIN = KIND == kStateRetention,
+                   BONUS = KIND == kStateBonus;
+    constexpr int NV = state_vectors(KIND), CW = kStateCW, NC = kStateNC, RG = 64 / CW, WV = CW * NC, WC = 4 * WV;
     constexpr int PER  = (TB * DQ * RG + 255) / 256;  // staged elements per vector and thread (dim <= DQ * RG)
     constexpr int VPER = (TB * WC + 255) / 256;
     static_assert(TB * TB <= 256, "one thread per token pair");
@@ -78,7 +108,7 @@ __global__ __launch_bounds__(256) void state_mix_kernel(StateMixParams p)
             S[ii][n] = (wave_on && pos0 > 0 && ii < dq) ? slab[(ii * NC + n) * 64 + lane] : 0.f;
         }
     }
-    const float  decay = LINEAR ? p.decay_h[h] : 0.f;
+    const float  decay = LINEAR || RETAIN ? p.decay_h[h] : 0.f;
     const int    tb    = min(TB, p.max_q_len);
     const size_t stage = (size_t)tb * (NV * Dp + WC);  // floats of one LDS buffer: [tb][NV][Dp] vectors, then [tb][WC] values
     float        rv[NV][PER], rval[VPER];
@@ -93,12 +123,21 @@ __global__ __launch_bounds__(256) void state_mix_kernel(StateMixParams p)
             const size_t row = (size_t)(row0 + t0 + t);
             const float* pr  = p.proj + row * p.ld + h * D + d;
             rv[0][r] = ok ? pr[p.c_q] : 0.f;
-            if constexpr (FORGET) {  // gate logit and lower bound; padding gets a gate of one: nothing is written there
+            if constexpr (RETAIN) {
+                const Rotation ro(p, pos0 + t0 + t, d);
+                rv[0][r] = ok ? ro(pr + p.c_q) : 0.f;
+                rv[1][r] = ok ? ro(pr + p.c_k) * p.k_mult : 0.f;
+            }
+            else             if constexpr (FORGET) {  // gate logit and lower bound; padding gets a gate of one: nothing is written there
                 rv[1][r] = ok ? pr[p.c_f] + p.f_bias[h * D + d] : 0.f;
                 rv[2][r] = ok ? p.f_low[h * D + d] : 1.f;
             }
             else {
                 rv[1][r] = ok ? pr[p.c_k] : 0.f;
+            }
+            if constexpr (BONUS) {
+                rv[2][r] = ok ? p.decay_w[row * p.ld_w + h * D + d] : 0.f;
+                rv[3][r] = ok ? p.bonus[h * D + d] : 0.f;
             }
             if constexpr (DELTA) {
                 rv[2][r] = ok ? p.decay_w[row * p.ld_w + h * D + d] : 0.f;
@@ -127,10 +166,16 @@ __global__ __launch_bounds__(256) void state_mix_kernel(StateMixParams p)
                     lds[(t * NV + 1) * Dp + d] = (1.f - low) * (z > 0.f ? lo : hi);              // 1 - f without cancellation
                     lds[(t * NV + 2) * Dp + d] = fmaf(1.f - low, z > 0.f ? hi : lo, low);        // f
                 }
+                else if constexpr (BONUS) {
+                    lds[(t * NV + 0) * Dp + d] = rv[0][r];
+                    lds[(t * NV + 1) * Dp + d] = rv[1][r];
+                    lds[(t * NV + 2) * Dp + d] = expf(-expf(rv[2][r]));
+                    lds[(t * NV + 3) * Dp + d] = rv[3][r] * rv[1][r];
+                }
                 else {
 #pragma unroll
                     for (int v = 0; v < NV; ++v) {
-                        lds[(t * NV + v) * Dp + d] = DELTA ? rv[v][r] : sm_silu(rv[v][r]);
+                        lds[(t * NV + v) * Dp + d] = DELTA || RETAIN ? rv[v][r] : sm_silu(rv[v][r]);
                     }
                 }
             }
@@ -307,8 +352,8 @@ __global__ __launch_bounds__(256) void state_mix_kernel(StateMixParams p)
             for (int t = 0; wave_on && t < nt; ++t) {
                 const float* q  = lds + (size_t)(t * NV + 0) * Dp + rg * dq;
                 const float* k  = lds + (size_t)(t * NV + 1) * Dp + rg * dq;
-                const float* w  = lds + (size_t)(t * NV + 2) * Dp + rg * dq;
-                const float* au = lds + (size_t)(t * NV + (DELTA ? 3 : 0)) * Dp + rg * dq;
+                const float* w  = lds + (size_t)(t * NV + (RETAIN ? 0 : 2)) * Dp + rg * dq;
+                const float* au = lds + (size_t)(t * NV + (DELTA || BONUS ? 3 : 0)) * Dp + rg * dq;  // a u, or bonus times key
                 const float* u  = lds + (size_t)(t * NV + (DELTA ? 4 : 0)) * Dp + rg * dq;
                 float        v[NC], us[NC], acc[NC];
 #pragma unroll
@@ -335,9 +380,14 @@ __global__ __launch_bounds__(256) void state_mix_kernel(StateMixParams p)
 #pragma unroll
                 for (int ii = 0; ii < DQ; ++ii) {
                     if (EXACT || ii < dq) {
-                        const float wv = w[ii], av = au[ii], kv = k[ii], qv = q[ii];
+                        const float wv = RETAIN ? decay : w[ii], av = au[ii], kv = k[ii], qv = q[ii];
 #pragma unroll
                         for (int n = 0; n < NC; ++n) {
+                            if constexpr (BONUS) {
+                                acc[n]   = fmaf(fmaf(av, v[n], S[ii][n]), qv, acc[n]);
+                                S[ii][n] = fmaf(wv, S[ii][n], kv * v[n]);
+                                continue;
+                            }
                             S[ii][n] = fmaf(wv, S[ii][n], DELTA ? fmaf(-av, us[n], kv * v[n]) : kv * v[n]);
                             acc[n]   = fmaf(S[ii][n], qv, acc[n]);
                         }
@@ -374,8 +424,8 @@ template<int KIND>
 static void launch_state_dq(const StateMixParams& p, dim3 grid, hipStream_t st)
 {
     const int  dp  = (p.dim + 7) / 8 * 8;
-    constexpr bool DELTA = KIND == kStateDelta, LINEAR = KIND == kStateLinear;
-    auto       lds = [&](int tb) { return (2 * (size_t)tb * ((DELTA ? 5 : LINEAR ? 2 : 3) * dp + 4 * kStateCW * kStateNC) + (LINEAR ? tb * tb : 0)) * sizeof(float); };
+    constexpr bool DELTA = KIND == kStateDelta, LINEAR = KIND == kStateLinear, CHUNKS = !DELTA && !LINEAR;
+    auto       lds = [&](int tb) { return (2 * (size_t)tb * (state_vectors(KIND) * dp + 4 * kStateCW * kStateNC) + (LINEAR ? tb * tb : 0)) * sizeof(float); };
     const bool one = p.max_q_len == 1;  // decoded tokens: one token per stage
 #define TM_STATE_LAUNCH_TB(DQ_, TB_)                                                     \
     if (p.dim == 8 * DQ_) {                                                              \
@@ -385,7 +435,7 @@ static void launch_state_dq(const StateMixParams& p, dim3 grid, hipStream_t st)
         state_mix_kernel<DQ_, KIND, TB_, false><<<grid, 256, lds(TB_), st>>>(p);        \
     }
 #define TM_STATE_LAUNCH(DQ_, TB_)                                             \
-    if constexpr (KIND == kStateForget) { /* one token: portions take chunks */ \
+    if constexpr (CHUNKS) { /* one token: portions take chunks */              \
         TM_STATE_LAUNCH_TB(DQ_, 1)                                            \
     }                                                                         \
     else if (one) {                                                           \
@@ -411,64 +461,81 @@ static void launch_state_dq(const StateMixParams& p, dim3 grid, hipStream_t st)
 #undef TM_STATE_LAUNCH_TB
 }
 
-// ---- forget-gate linear attention over prompt portions: chunks of 16 tokens on the fp32 matrix cores ------------------------------------
+// ---- linear attention with decays over prompt portions: chunks of 16 tokens on the fp32 matrix cores -------------------------------------
+// Serves the forget-gate mixer (k = 1 - f), retention (f = the head's decay, q and k rotated as they are loaded) and the bonus recurrence.
 // Per chunk, head and key channel d, with t, j counting tokens of the chunk and P(a..b) = prod of f_s[d] for a <= s <= b:
-//   o_t = sum_d q_t P(0..t) S0[d] + sum_{j <= t} A[t][j] v_j,    A[t][j] = sum_d q_t k_j P(j+1..t),    k = 1 - f
+//   o_t = sum_d q_t P(0..t) S0[d] + sum_{j <= t} A[t][j] v_j,    A[t][j] = sum_d q_t k_j P(j+1..t)
 //   S   = P(0..15) S0 + sum_j k_j P(j+1..15) v_j^T
+// The bonus recurrence reads the state ahead of its token: P(0..t-1) and P(j+1..t-1) in o_t and A[t][j < t], and A[t][t] = sum_d q_t u k_t.
 // Every factor is a running product of numbers in [0, 1]: nothing is divided by a decay, so gates near zero cost no precision.
-//   forget_blocks_kernel: everything that does not depend on the state -- scaled queries, scaled keys, A, the chunk's whole decay -- for all
+//   decay_blocks_kernel: everything that does not depend on the state -- scaled queries, scaled keys, A, the chunk's whole decay -- for all
 //                         chunks of the launch at once, one workgroup per (chunk, head), written in the order the second kernel's MFMA operands are read
-//   forget_chunks_kernel: a wave owns 16 value columns of a head's state in MFMA accumulators and walks the sequence's chunks; the
+//   decay_chunks_kernel: a wave owns 16 value columns of a head's state in MFMA accumulators and walks the sequence's chunks; the
 //                         accumulator layout (row = lane / 16 * 4 + i) serves as the B operand of the query product as it is, the
 //                         contraction index runs over (row tile, i) with lane group g on row 16 r + 4 g + i
 // v_mfma_f32_16x16x4_f32: full 32-bit products and sums.  Block of a (chunk, head), DR = ceil(dim / 16) row tiles, floats:
 //   scaled queries [DR][64 lanes][4], scaled keys [DR][64][4], A [64][4], chunk decay [DR * 16]
 constexpr int kChunkT = 16;
 
-__host__ __device__ inline int forget_tiles(int dim)  // row tiles of an instantiation
+__host__ __device__ inline int decay_tiles(int dim)  // row tiles of an instantiation
 {
     const int n = (dim + 15) / 16;
     return n <= 2 ? 2 : n <= 4 ? 4 : n <= 8 ? 8 : 16;
 }
-__host__ __device__ inline size_t forget_block_floats(int dim)
+__host__ __device__ inline size_t decay_block_floats(int dim)
 {
-    const int dr = forget_tiles(dim);
+    const int dr = decay_tiles(dim);
     return (size_t)dr * 64 * 4 * 2 + 256 + dr * 16;
 }
 // chunk c of sequence s, whose first row is row0 of the launch: sequences take (rows before) / 16 + s onwards, which never overlaps
-__device__ __forceinline__ size_t forget_chunk_index(int s, int row0, int c)
+__device__ __forceinline__ size_t decay_chunk_index(int s, int row0, int c)
 {
     return (size_t)(row0 / kChunkT + s + c);
 }
 
-size_t forget_workspace_floats(int rows, int nseq, int heads, int dim)
+size_t decay_workspace_floats(int rows, int nseq, int heads, int dim)
 {
-    return ((size_t)rows / kChunkT + nseq + 1) * heads * forget_block_floats(dim);
+    return ((size_t)rows / kChunkT + nseq + 1) * heads * decay_block_floats(dim);
 }
 
 // grid (nseq * chunks, heads), 256 threads
-template<int DR>
-__global__ __launch_bounds__(256) void forget_blocks_kernel(StateMixParams p, int chunks)
+template<int DR, int KIND>
+__global__ __launch_bounds__(256) void decay_blocks_kernel(StateMixParams p, int chunks)
 {
     constexpr int DP = DR * 16, LD = DP + 4, NM = (DP + 63) / 64;
     __shared__ __attribute__((aligned(16))) float sq[kChunkT * LD], sk[kChunkT * LD], sf[kChunkT * LD];
+    constexpr bool FORGET = KIND == kStateForget, RETAIN = KIND == kStateRetention, BONUS = KIND == kStateBonus;
     const int s = blockIdx.x / chunks, c = blockIdx.x % chunks, h = blockIdx.y, D = p.dim, tid = threadIdx.x;
     const int row0 = p.cu_q[s] - p.cu_q[0], q_len = p.cu_q[s + 1] - p.cu_q[s];
     const int t0 = c * kChunkT, nt = min(kChunkT, q_len - t0);
     if (nt <= 0) {
         return;
     }
-    float* out = p.blocks + (forget_chunk_index(s, row0, c) * p.heads + h) * forget_block_floats(D);
+    float* out = p.blocks + (decay_chunk_index(s, row0, c) * p.heads + h) * decay_block_floats(D);
     for (int i = tid; i < kChunkT * DP; i += 256) {
         const int  t = i / DP, d = i % DP;
         float      q = 0.f, k = 0.f, f = 1.f;  // tokens behind the portion and channels behind dim: nothing read, nothing written, nothing forgotten
         if (t < nt && d < D) {
-            const float* pr = p.proj + (size_t)(row0 + t0 + t) * p.ld + h * D + d;
-            const float  z = pr[p.c_f] + p.f_bias[h * D + d], low = p.f_low[h * D + d];
-            const float  ez = expf(-fabsf(z)), hi = 1.f / (1.f + ez), lo = ez * hi;  // sigmoid(|z|), sigmoid(-|z|)
-            q = sm_silu(pr[p.c_q]);
-            k = (1.f - low) * (z > 0.f ? lo : hi);
-            f = fmaf(1.f - low, z > 0.f ? hi : lo, low);
+            const size_t row = (size_t)(row0 + t0 + t);
+            const float* pr  = p.proj + row * p.ld + h * D + d;
+            if constexpr (FORGET) {
+                const float z = pr[p.c_f] + p.f_bias[h * D + d], low = p.f_low[h * D + d];
+                const float ez = expf(-fabsf(z)), hi = 1.f / (1.f + ez), lo = ez * hi;  // sigmoid(|z|), sigmoid(-|z|)
+                q = sm_silu(pr[p.c_q]);
+                k = (1.f - low) * (z > 0.f ? lo : hi);
+                f = fmaf(1.f - low, z > 0.f ? hi : lo, low);
+            }
+            else if constexpr (RETAIN) {
+                const Rotation ro(p, p.k_len[s] - q_len + t0 + t, d);
+                q = ro(pr + p.c_q);
+                k = ro(pr + p.c_k) * p.k_mult;
+                f = p.decay_h[h];
+            }
+            else {
+                q = pr[p.c_q];
+                k = pr[p.c_k];
+                f = expf(-expf(p.decay_w[row * p.ld_w + h * D + d]));
+            }
         }
         sq[t * LD + d] = q;
         sk[t * LD + d] = k;
@@ -494,8 +561,14 @@ __global__ __launch_bounds__(256) void forget_blocks_kernel(StateMixParams p, in
                     const floatx4 q = *(const floatx4*)(sq + t * LD + d), f = *(const floatx4*)(sf + t * LD + d);
 #pragma unroll
                     for (int i = 0; i < 4; ++i) {
-                        w[m][i] *= t > j ? f[i] : 1.f;
-                        dot = fmaf(q[i], w[m][i], dot);
+                        if constexpr (BONUS) {  // the key meets its own token through the bonus, and decays behind each later one
+                            dot = fmaf(q[i], t == j && d + i < D ? w[m][i] * p.bonus[h * D + d + i] : w[m][i], dot);
+                            w[m][i] *= t > j ? f[i] : 1.f;
+                        }
+                        else {
+                            w[m][i] *= t > j ? f[i] : 1.f;
+                            dot = fmaf(q[i], w[m][i], dot);
+                        }
                     }
                 }
             }
@@ -512,8 +585,14 @@ __global__ __launch_bounds__(256) void forget_blocks_kernel(StateMixParams p, in
         if (i < DP) {
 #pragma unroll
             for (int t = 0; t < kChunkT; ++t) {
-                run *= sf[t * LD + d];
-                sq[t * LD + d] *= run;
+                if constexpr (BONUS) {
+                    sq[t * LD + d] *= run;
+                    run *= sf[t * LD + d];
+                }
+                else {
+                    run *= sf[t * LD + d];
+                    sq[t * LD + d] *= run;
+                }
             }
             out[DR * 64 * 4 * 2 + 256 + d] = run;
         }
@@ -540,7 +619,7 @@ __global__ __launch_bounds__(256) void forget_blocks_kernel(StateMixParams p, in
 
 // grid (nseq, heads, ceil(vdim / 64)), 256 threads: wave -> 16 value columns
 template<int DR>
-__global__ __launch_bounds__(256) void forget_chunks_kernel(StateMixParams p)
+__global__ __launch_bounds__(256) void decay_chunks_kernel(StateMixParams p)
 {
     constexpr int NC = kStateNC, WV = kStateCW * kStateNC;
     const int s = blockIdx.x, h = blockIdx.y, lane = threadIdx.x & 63, cb = blockIdx.z * 4 + (threadIdx.x >> 6);
@@ -566,8 +645,8 @@ __global__ __launch_bounds__(256) void forget_chunks_kernel(StateMixParams p)
             S[r][i]     = pos0 > 0 && d < D ? slab[at(d)] : 0.f;
         }
     }
-    const size_t bf  = forget_block_floats(D);
-    const float* blk = p.blocks + (forget_chunk_index(s, row0, 0) * p.heads + h) * bf;
+    const size_t bf  = decay_block_floats(D);
+    const float* blk = p.blocks + (decay_chunk_index(s, row0, 0) * p.heads + h) * bf;
     struct Operands {
         floatx4 q[DR], k[DR], f[DR], a, v;
     };
@@ -657,23 +736,24 @@ __global__ __launch_bounds__(256) void forget_chunks_kernel(StateMixParams p)
     }
 }
 
-static int launch_forget_chunks(const StateMixParams& p, hipStream_t st)
+template<int KIND>
+static int launch_decay_chunks(const StateMixParams& p, hipStream_t st)
 {
-    TM_REQUIRE(p.blocks && p.blocks_floats >= forget_workspace_floats(p.rows, p.nseq, p.heads, p.dim), "state mixer: chunk workspace");
+    TM_REQUIRE(p.blocks && p.blocks_floats >= decay_workspace_floats(p.rows, p.nseq, p.heads, p.dim), "state mixer: chunk workspace");
     const int  chunks = (p.max_q_len + kChunkT - 1) / kChunkT;
     const dim3 gb(p.nseq * chunks, p.heads), gc(p.nseq, p.heads, (p.vdim + 63) / 64);
-#define TM_FORGET(DR_)                                           \
-    case DR_:                                                    \
-        forget_blocks_kernel<DR_><<<gb, 256, 0, st>>>(p, chunks); \
-        forget_chunks_kernel<DR_><<<gc, 256, 0, st>>>(p);        \
+#define TM_CHUNKS(DR_)                                                  \
+    case DR_:                                                           \
+        decay_blocks_kernel<DR_, KIND><<<gb, 256, 0, st>>>(p, chunks); \
+        decay_chunks_kernel<DR_><<<gc, 256, 0, st>>>(p);               \
         break;
-    switch (forget_tiles(p.dim)) {
-        TM_FORGET(2)
-        TM_FORGET(4)
-        TM_FORGET(8)
-        TM_FORGET(16)
+    switch (decay_tiles(p.dim)) {
+        TM_CHUNKS(2)
+        TM_CHUNKS(4)
+        TM_CHUNKS(8)
+        TM_CHUNKS(16)
     }
-#undef TM_FORGET
+#undef TM_CHUNKS
     TM_HIP_CHECK(hipGetLastError());
     return 0;
 }
@@ -683,13 +763,22 @@ int launch_state_mix(const StateMixParams& p, int kind, hipStream_t st)
     TM_REQUIRE(p.nseq >= 0 && p.heads >= 1 && p.dim >= 1 && p.dim <= 256 && p.vdim >= 1 && p.max_q_len >= 1, "state mixer: sizes (dim <= 256)");
     TM_REQUIRE(p.cu_q && p.k_len && p.state && p.proj && p.out && p.ld >= 1 && p.ldo >= p.heads * p.vdim, "state mixer: operands");
     TM_REQUIRE(kind == kStateDelta ? (p.decay_w && p.unit && p.ld_w >= p.heads * p.dim && p.ld_u >= p.heads * p.dim) :
-               kind == kStateForget ? (p.f_bias && p.f_low) : (kind == kStateLinear && p.decay_h),
+               kind == kStateForget ? (p.f_bias && p.f_low) :
+               kind == kStateBonus ? (p.decay_w && p.bonus && p.ld_w >= p.heads * p.dim) : ((kind == kStateLinear || kind == kStateRetention) && p.decay_h),
                "state mixer: decay operands");
     if (p.nseq == 0) {
         return 0;
     }
-    if (kind == kStateForget && p.max_q_len > 1) {
-        return launch_forget_chunks(p, st);
+    TM_REQUIRE(kind != kStateRetention || (p.rot_dims >= 0 && p.rot_dims % 2 == 0 && p.rot_dims <= p.dim && (p.rot_dims == 0 || p.inv_freq)),
+               "state mixer: rotation");
+    if (p.max_q_len > 1 && kind == kStateForget) {
+        return launch_decay_chunks<kStateForget>(p, st);
+    }
+    if (p.max_q_len > 1 && kind == kStateRetention) {
+        return launch_decay_chunks<kStateRetention>(p, st);
+    }
+    if (p.max_q_len > 1 && kind == kStateBonus) {
+        return launch_decay_chunks<kStateBonus>(p, st);
     }
     const int  wcols = 4 * kStateCW * kStateNC;  // value columns of a workgroup
     const dim3 grid(p.nseq, p.heads, (p.vdim + wcols - 1) / wcols);
@@ -698,6 +787,12 @@ int launch_state_mix(const StateMixParams& p, int kind, hipStream_t st)
     }
     else if (kind == kStateForget) {
         launch_state_dq<kStateForget>(p, grid, st);
+    }
+    else if (kind == kStateRetention) {
+        launch_state_dq<kStateRetention>(p, grid, st);
+    }
+    else if (kind == kStateBonus) {
+        launch_state_dq<kStateBonus>(p, grid, st);
     }
     else {
         launch_state_dq<kStateLinear>(p, grid, st);
@@ -887,11 +982,19 @@ int launch_short_conv(float* y, int ldy, const float* x, int ldx, int x_col, con
 template<class T>
 __global__ __launch_bounds__(256) void gated_group_norm_kernel(T* __restrict__ y, int ldy, const float* __restrict__ x, int ldx,
                                                                const float* __restrict__ w, const float* __restrict__ gate, int ldg, int groups,
-                                                               int n, float eps)
+                                                               int n, float eps, int silu, float mult)
 {
     __shared__ float red[4];
     const int    t = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const float* xr = x + (size_t)t * ldx;
+    auto close = [&](float o, size_t c) {  // weight, gate, factor
+        o *= w ? w[c] : 1.f;
+        if (gate) {
+            const float g = gate[(size_t)t * ldg + c];
+            o             = (silu ? o * g : o) / (1.f + expf(-g));
+        }
+        return o * mult;
+    };
     if (groups == 1) {
         float ss = 0.f;
         for (int i = threadIdx.x; i < n; i += 256) {
@@ -904,8 +1007,7 @@ __global__ __launch_bounds__(256) void gated_group_norm_kernel(T* __restrict__ y
         __syncthreads();
         const float inv = 1.0f / sqrtf(((red[0] + red[1]) + (red[2] + red[3])) / (float)n + eps);
         for (int i = threadIdx.x; i < n; i += 256) {
-            const float o          = xr[i] * inv * w[i];
-            y[(size_t)t * ldy + i] = (T)(gate ? o / (1.f + expf(-gate[(size_t)t * ldg + i])) : o);
+            y[(size_t)t * ldy + i] = (T)close(xr[i] * inv, i);
         }
         return;
     }
@@ -918,24 +1020,23 @@ __global__ __launch_bounds__(256) void gated_group_norm_kernel(T* __restrict__ y
         const float inv = 1.0f / sqrtf(group_sum<64>(ss) / (float)n + eps);
         for (int i = lane; i < n; i += 64) {
             const size_t c = (size_t)g * n + i;
-            const float  o = xg[i] * inv * w[c];
-            y[(size_t)t * ldy + c] = (T)(gate ? o / (1.f + expf(-gate[(size_t)t * ldg + c])) : o);
+            y[(size_t)t * ldy + c] = (T)close(xg[i] * inv, c);
         }
     }
 }
 
 int launch_gated_group_norm(void* y, int ldy, int out_elem_bytes, const float* x, int ldx, const float* w, const float* gate, int ldg, int rows,
-                            int groups, int n, float eps, hipStream_t st)
+                            int groups, int n, float eps, hipStream_t st, bool silu, float mult)
 {
-    TM_REQUIRE(y && x && w && groups >= 1 && n >= 1 && ldy >= groups * n && ldx >= groups * n && (!gate || ldg >= groups * n), "gated norm: operands");
+    TM_REQUIRE(y && x && groups >= 1 && n >= 1 && ldy >= groups * n && ldx >= groups * n && (!gate || ldg >= groups * n), "gated norm: operands");
     if (rows == 0) {
         return 0;
     }
     if (out_elem_bytes == 2) {
-        gated_group_norm_kernel<__bf16><<<rows, 256, 0, st>>>((__bf16*)y, ldy, x, ldx, w, gate, ldg, groups, n, eps);
+        gated_group_norm_kernel<__bf16><<<rows, 256, 0, st>>>((__bf16*)y, ldy, x, ldx, w, gate, ldg, groups, n, eps, silu, mult);
     }
     else {
-        gated_group_norm_kernel<float><<<rows, 256, 0, st>>>((float*)y, ldy, x, ldx, w, gate, ldg, groups, n, eps);
+        gated_group_norm_kernel<float><<<rows, 256, 0, st>>>((float*)y, ldy, x, ldx, w, gate, ldg, groups, n, eps, silu, mult);
     }
     TM_HIP_CHECK(hipGetLastError());
     return 0;

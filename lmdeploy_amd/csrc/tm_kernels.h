@@ -347,7 +347,7 @@ enum { kDenseBf16 = 0, kDenseF32 = 1 };
 // y = act(acc) * table[ids[m]][table_col + n] (activation type; one row of a bf16 table per output row, chosen by its token id)
 // y = xielu(acc) (activation type; act_par = {softplus(p), 1/2 + softplus(q)}: z > 0: a z^2 + z / 2, else b (e^z - 1 - z) + z / 2)
 enum { kDenseStore = 0, kDenseRelu2 = 1, kDenseResidAdd = 2, kDenseScaleF32 = 3, kDenseBiasF32 = 4, kDenseResidGate = 5, kDenseGatedAct = 6, kDenseXielu = 7, kDenseActTable = 8 };
-enum { kActRelu2 = 0, kActGeluTanh = 1, kActSilu = 2, kActXielu = 3 };  // (= TM_ACT_*)
+enum { kActRelu2 = 0, kActGeluTanh = 1, kActSilu = 2, kActXielu = 3, kActClamped = 5 };  // (= TM_ACT_*)
 __device__ __forceinline__ float act_apply(int act, float z)
 {
     if (act == kActGeluTanh) {
@@ -369,6 +369,7 @@ inline int dense_pair_rows(int n_out)  // rows of a paired image for n_out outpu
 {
     return (n_out + 15) / 16 * 32;
 }
+constexpr int kDenseMaxSeg = 8;
 struct DenseWeight {
     int    K = 0, N = 0, Kp = 0, Np = 0;  // Kp = K rounded up to 32, Np = N rounded up to 128: zero-padded image [Np][Kp]
     int    dtype = kDenseBf16;
@@ -391,6 +392,10 @@ struct DenseCall {
     const int*   ids = nullptr;
     int          ld_table = 0, table_col = 0, table_rows = 0;
     int          act = kActRelu2, n_out = 0;  // kDenseGatedAct: the activation and the number of outputs (the image has 2 rows per output)
+    float        act_limit = 0.f, act_alpha = 0.f;  // kActClamped: g = min(gate, limit), u = clamp(up, +-limit), y = g sigmoid(alpha g) (u + 1)
+    // count == 1: the output columns [seg_n0[i], seg_n0[i + 1]) read x at column i * x_col_stride -- projections of several inputs of a row in
+    // one launch (seg_n0[0] = 0, every border a multiple of 128; n_seg = 0: one input)
+    int          n_seg = 0, seg_n0[kDenseMaxSeg] = {};
     int          count = 1;             // items; item g uses image g, x column g * x_col_stride, y column g * y_col_stride ...
     int          x_col_stride = 0, y_col_stride = 0;
     const int*   row_offsets = nullptr; // ... and, when set, the rows [row_offsets[g], row_offsets[g + 1]) of x and y (device, [count + 1])
@@ -483,6 +488,7 @@ struct AttnPrepExtra {
     int          rot_dims = 0;
     int          maps = 1, rot_pairs = 0;
     float        rot_mult = 1.f;
+    float        v_mult = 1.f;  // the values are stored times v_mult (the attention output is linear in them)
     // conv_w != nullptr (launches with ONE row per sequence: decoded tokens): the source columns first pass the short causal convolution
     // of launch_short_conv in this kernel -- column c is channel c of conv_w [conv_ch][conv_taps] and of the sequence's state
     // [conv_taps - 1][conv_ch] at conv_state + slot * conv_slot_stride + conv_offset, which the wave that owns a channel reads and rewrites
@@ -523,11 +529,18 @@ int launch_concat2(void* out, int ldo, int out_elem_bytes, const float* a, const
 int launch_moe_topk_sigmoid(int* ids, float* w, const float* logits, int ld, int T, int E, int k, hipStream_t st);
 // soft-max over all E logits; the k largest scores win (ties: the lower index); w = scale * score (not renormalised)
 int launch_moe_topk_softmax(int* ids, float* w, const float* logits, int ld, int T, int E, int k, float scale, hipStream_t st);
+// scores s = sigmoid(logit); experts are ordered by s + correction[e] (nullptr: by s) and come from the `keep` best of `groups` equal groups of
+// neighbours, a group counting the sum of its two best (ties: the lower index); w = the chosen s, divided by their sum + 1e-20 with renorm
+int launch_moe_topk_grouped(int* ids, float* w, const float* logits, int ld, const float* correction, int T, int E, int groups, int keep, int k,
+                            bool renorm, hipStream_t st);
+// shared_offsets != nullptr: behind the T k routed rows follow all T rows once more, unscaled (an expert that every token visits, item E of the
+// batched products), and shared_offsets[E + 1] = T (k + 1) is written
 int launch_moe_gather(void* xs, int lds, const void* x, int ldx, int elem_bytes, const float* w, const int* en2f, int T, int H, int k, bool scale,
-                      hipStream_t st);
+                      hipStream_t st, int* shared_offsets = nullptr, int E = 0);
 int launch_moe_combine_f32(float* resid, const float* y, const float* w, const int* en2f, const float* gate, int ldg, const float* gate_bias, int T,
                            int H, int k, bool weighted, hipStream_t st, bool overwrite = false /* resid = sum instead of resid += sum */,
-                           const float* add = nullptr /* overwrite: resid = add + sum ([T][H]) */);
+                           const float* add = nullptr /* overwrite: resid = add + sum ([T][H]) */,
+                           const float* add_gate = nullptr /* ... add[t] times sigmoid(add_gate[t * ld_add_gate]) */, int ld_add_gate = 0);
 // offsets[n + 1] = offsets[n] + extra: one more item behind the n items of a routing table (rows that every token sends)
 int launch_moe_extend_offsets(int* offsets, int n, int extra, hipStream_t st);
 // layer norm with bias on the fp32 stream.  launch_layernorm_f32: y[m] = LN(x[rows ? rows[m] : m]) (bf16 | fp32 [M][ldy]);
@@ -584,17 +597,48 @@ struct StateMixParams {
     const float* decay_w = nullptr;   // delta: [rows][ld_w] decay per key channel
     const float* unit = nullptr;      // delta: [rows][ld_u] unit keys
     int          ld_w = 0, ld_u = 0;
+    const float* inv_freq = nullptr;  // retention: queries and keys turn in their first rot_dims channels (channel i with i + rot_dims / 2) by
+    int          rot_dims = 0;        // position * inv_freq[i]; keys are then multiplied by k_mult
+    float        k_mult = 1.f;
+    const float* bonus = nullptr;     // bonus recurrence: [heads * dim]; its decays are exp(-exp(decay_w))
     int          c_f = 0;             // forget gate: column of its logits; f = low + (1 - low) sigmoid(logit + bias) decays and 1 - f is the key
     const float *f_bias = nullptr, *f_low = nullptr;  // [heads * dim]
-    int          rows = 0;            // forget gate, max_q_len > 1: rows of the launch, and scratch of forget_workspace_floats()
+    int          rows = 0;            // mixers in chunks, max_q_len > 1: rows of the launch, and scratch of decay_workspace_floats()
     float*       blocks = nullptr;
     size_t       blocks_floats = 0;
     float*       out = nullptr;       // [rows][ldo] fp32, head h at h * vdim
     int          ldo = 0;
 };
+// several inputs made of a token's row h and its predecessor's h' (zeros ahead of the sequence): mix s = h + (h' - h) mu[s], s < n_mix, at column
+// (1 + s) * mix_stride of row m of `out` ([.][ld], bf16 | fp32; column 0 is h itself, written by whoever made h).  The last row of a sequence is state
+// (H floats at seqs.layer_offset of the slot)
+struct TokenShift {
+    int            n_mix = 0;
+    const float*   mu = nullptr;      // [n_mix][H]
+    void*          out = nullptr;
+    int            ld = 0, mix_stride = 0, elem_bytes = 2;
+    StateMixParams seqs;
+};
+// prompt portions: h fp32 [rows][H] (the part's first row first), row_seq / row_pos of its rows
+int launch_token_shift(const float* h, const TokenShift& s, const int* row_seq, const int* row_pos, int rows, int H, hipStream_t st);
+// the end of a sublayer between two RMS norms, one workgroup per row.  v = x[m] (+ y[m] / rms(y[m]) * (w_offset + post_w) with y) (+ x0[m] with x0);
+// x[m] = v; with next_w: h[m] = v / rms(v) * (w_offset + next_w) in the activation type, with hf also in fp32 ([M][H]).  shift.n_mix > 0: the rows
+// [0, shift_rows) are decoded tokens (row m = sequence m of shift.seqs): their mixes are formed here and their state is updated
+struct BlockClose {
+    float*       x = nullptr;
+    const float *y = nullptr, *post_w = nullptr, *x0 = nullptr, *next_w = nullptr;
+    void*        h = nullptr;
+    int          ldh = 0, h_elem_bytes = 2;
+    float*       hf = nullptr;
+    float        w_offset = 0.f, eps = 0.f;
+    int          M = 0, H = 0;
+    int          shift_rows = 0;
+    TokenShift   shift;
+};
+int    launch_block_close(const BlockClose& c, hipStream_t st);
 size_t state_mix_floats(int heads, int dim, int vdim);  // floats of one layer's state in one slot
-size_t forget_workspace_floats(int rows, int nseq, int heads, int dim);
-enum { kStateLinear = 0, kStateDelta = 1, kStateForget = 2 };
+size_t decay_workspace_floats(int rows, int nseq, int heads, int dim);
+enum { kStateLinear = 0, kStateDelta = 1, kStateForget = 2, kStateRetention = 3, kStateBonus = 4 };
 int    launch_state_mix(const StateMixParams& p, int kind, hipStream_t st);
 int    launch_delta_prep(float* proj, int ld, int c_k, int c_a, float* decay, int ld_w, float* unit, int ld_u, int rows, int heads, int dim,
                          hipStream_t st);
@@ -610,9 +654,9 @@ int    launch_gdelta_prep(float* src, int ld, int c_q, int c_k, int c_qo, int c_
 // StateMixParams (cu_q, k_len, seq_slot / slot0, active / park_slot, state, slot_stride, layer_offset)
 int    launch_short_conv(float* y, int ldy, const float* x, int ldx, int x_col, const float* w, int channels, int taps, int act,
                          const StateMixParams& seqs, hipStream_t st);
-// (gate == nullptr: no gate)
+// (gate == nullptr: no gate; w == nullptr: no weight; silu: the gate is silu(gate) instead of sigmoid(gate); mult: a factor on the result)
 int    launch_gated_group_norm(void* y, int ldy, int out_elem_bytes, const float* x, int ldx, const float* w, const float* gate, int ldg, int rows,
-                               int groups, int n, float eps, hipStream_t st);
+                               int groups, int n, float eps, hipStream_t st, bool silu = false, float mult = 1.f);
 // y[row][h n + i] = o / sqrt(mean_i(o^2) + eps) * mult, o = a[row][h n + i] - lambda[0] * a[row][(heads + h) n + i]: the two maps of
 // differential attention (map-major heads, fp32) joined per head
 int launch_diff_head_norm(void* y, int ldy, int out_elem_bytes, const float* a, int lda, const float* lambda, float mult, int rows, int heads, int n,

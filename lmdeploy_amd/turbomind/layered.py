@@ -25,9 +25,9 @@ import numpy as np
 from .. import _ffi
 from .engine import Engine
 
-MIXER_ATTENTION, MIXER_LATENT, MIXER_LIGHTNING, MIXER_DELTA, MIXER_PARALLEL, MIXER_FORGET = 1, 2, 3, 4, 5, 6
+MIXER_ATTENTION, MIXER_LATENT, MIXER_LIGHTNING, MIXER_DELTA, MIXER_PARALLEL, MIXER_FORGET, MIXER_RETENTION = 1, 2, 3, 4, 5, 6, 7
 MLP_NONE, MLP_DENSE, MLP_GATED, MLP_MOE = 0, 1, 2, 3
-ACT_RELU2, ACT_GELU_TANH, ACT_SILU, ACT_XIELU, ACT_POLYNORM = 0, 1, 2, 3, 4
+ACT_RELU2, ACT_GELU_TANH, ACT_SILU, ACT_XIELU, ACT_POLYNORM, ACT_CLAMPED = 0, 1, 2, 3, 4, 5
 DTYPES = {'bfloat16': 0, 'bf16': 0, 'float32': 1, 'f32': 1}
 
 
@@ -94,6 +94,16 @@ class LayerSpec:
     pre_norm: bool = False        # x += mixer(LN1 x); x += ff(LN2 x), layer norms with bias
     q_rank: int = 0               # latent attention: > 0: the queries go through a normed latent of this size
     kv_from: int = -1             # latent attention: >= 0: attends over what that layer has cached
+    both_norms: bool = False      # x += N(mixer(N x)); x += N(ff(N x)): an RMS norm ahead of and behind each sublayer
+    left_scale: float = 1.0       # parallel pair in such a block: weights of the two mixers' results
+    right_scale: float = 1.0
+    act_limit: float = 0.0        # clamped gated feed-forward: bound of gate and up, factor inside the sigmoid
+    act_alpha: float = 0.0
+    group_count: int = 0          # routed experts: equal groups of neighbours, and how many of them may be chosen from
+    group_keep: int = 0
+    router_correction: bool = False  # a learned number per expert joins its score when experts are ordered
+    router_renorm: bool = False   # the chosen scores are divided by their sum
+    shared_gate: bool = False     # the shared expert's result times a sigmoid of one number per token
 
 
 @dataclass
@@ -114,6 +124,8 @@ class LayeredConfig:
     logit_softcap: float = 0.0    # > 0: logits <- cap * tanh(logits / cap)
     norm_groups: int = 0          # > 0: the last norm is an RMS norm in that many groups
     side_dim: int = 0             # > 0: every layer reads a part of this size of a second embedding table by the token id
+    loop_add: bool = False        # the embedding output joins the stream ahead of every pass of the loop but the first
+    tied_head: bool = False       # the logits come from the embedding table
     depth_avg: bool = False       # a layer hands on a learned average of the embedding output and all results so far
     names: list = field(default_factory=list)   # tensor prefix of every layer run with tensors of its own ('' -> 'l<index>.')
 
@@ -135,11 +147,14 @@ class LayeredConfig:
                            int(s.expert_plain), int(s.router_softmax), s.router_scale, s.shared_ff,
                            s.norm_groups, s.conv_taps, int(s.diff_maps), s.diff_init, int(s.rot_pairs), s.yarn_factor, s.yarn_original, s.yarn_fast,
                            s.yarn_slow, s.dist_buckets, s.dist_max, s.r_heads, s.r_kv_heads, s.r_dim, s.r_vdim, s.r_conv, s.a_rank, s.g_rank,
-                           int(s.pre_norm), s.q_rank, s.kv_from)
+                           int(s.pre_norm), s.q_rank, s.kv_from,
+                           int(s.both_norms), s.left_scale, s.right_scale, s.act_limit, s.act_alpha, s.group_count, s.group_keep,
+                           int(s.router_correction), int(s.router_renorm), int(s.shared_gate))
             for s in self.layers])
         return _ffi.LayeredConfig(self.width, self.vocab, len(self.layers), arr, self.norm_eps, self.norm_offset, self.residual_mult,
                                   self.logit_scale, DTYPES[dtype], self.loop_times, int(self.final_layer_norm), self.embed_scale,
-                                  self.logit_softcap, self.norm_groups, self.side_dim, int(self.depth_avg)), (arr, keep)
+                                  self.logit_softcap, self.norm_groups, self.side_dim, int(self.depth_avg), int(self.loop_add),
+                                  int(self.tied_head)), (arr, keep)
 
     def tensor_name(self, run: int, leaf: str) -> str:
         """checkpoint name of tensor `leaf` of layer run `run` (the engine's slots count layer RUNS; a looped model's file counts layers)"""
@@ -147,7 +162,9 @@ class LayeredConfig:
 
     def tensor_shapes(self) -> dict:
         """{tensor name: shape} a checkpoint of this config holds"""
-        W, out = self.width, {'embed': (self.vocab, self.width), 'final.norm': (self.width,), 'head': (self.vocab, self.width)}
+        W, out = self.width, {'embed': (self.vocab, self.width), 'final.norm': (self.width,)}
+        if not self.tied_head:
+            out['head'] = (self.vocab, W)
         if self.final_layer_norm and not self.norm_groups:
             out['final.norm.b'] = (W,)
         if self.loop_times > 0:
@@ -165,6 +182,9 @@ class LayeredConfig:
                     out[p + 'side.gate'], out[p + 'side.proj'], out[p + 'side.norm'] = (self.side_dim, W), (W, self.side_dim), (W,)
                 if self.depth_avg:
                     out[p + 'dwa'] = (i + 2,)
+                continue
+            if s.both_norms:
+                out.update(_both_shapes(p, s, W))
                 continue
             if s.post_norm and s.norm_groups:
                 out.update(_group_shapes(p, s, W))
@@ -305,6 +325,147 @@ def _pre_shapes(p: str, s: LayerSpec, W: int) -> dict:
         if s.act == ACT_POLYNORM:
             out[p + 'mlp.act'] = (4,)
     return out
+
+
+def _both_shapes(p: str, s: LayerSpec, W: int) -> dict:
+    """tensors of a block with an RMS norm ahead of and behind each sublayer: retention, or the parallel pair of a convolved windowed
+    attention and a time mixer; clamped gated feed-forward, or grouped experts with a gated shared one"""
+    H, G, d, dv = s.heads, s.kv_heads, s.dim, s.vdim
+    out = {p + 'norm1b': (W,)}
+    if s.mixer == MIXER_RETENTION:
+        for t, n in (('q', H * d), ('k', H * d), ('v', H * dv), ('g', H * dv)):
+            out[p + 'mix.' + t] = (n, W)
+        out[p + 'mix.o'] = (W, H * dv)
+    elif s.mixer == MIXER_PARALLEL:
+        a, b, n_r = p + 'mix.left.', p + 'mix.right.', s.r_heads * s.r_dim
+        for t, n in (('q', H * d), ('k', G * d), ('v', G * dv)):
+            out[a + t] = (n, W)
+            if s.conv_taps:
+                out[a + t + '.conv'] = (n, s.conv_taps)
+        if s.sink:
+            out[a + 'sink'] = (H,)
+        out[a + 'o'] = (W, H * dv)
+        for t in 'rkvgw':
+            out[b + 'mu.' + t] = (W,)
+        for t in 'rkvg':
+            out[b + t] = (n_r, W)
+        out.update({b + 'w1': (s.decay_rank, W), b + 'w2': (n_r, s.decay_rank), b + 'w0': (n_r,), b + 'u': (s.r_heads, s.r_dim), b + 'norm': (n_r,),
+                    b + 'o': (W, n_r)})
+    else:
+        raise NotImplementedError(f'{p}: mixer {s.mixer} in a block with norms on both sides')
+    if s.mlp:
+        out[p + 'norm2'], out[p + 'norm2b'] = (W,), (W,)
+    if s.mlp == MLP_GATED:
+        out[p + 'mlp.gate'], out[p + 'mlp.up'], out[p + 'mlp.down'] = (s.ff, W), (s.ff, W), (W, s.ff)
+    elif s.mlp == MLP_MOE:
+        out[p + 'mlp.router'] = (s.experts, W)
+        if s.router_correction:
+            out[p + 'mlp.correction'] = (s.experts,)
+        for e, ff in [(f'e{e}', s.ff) for e in range(s.experts)] + ([('shared', s.shared_ff)] if s.shared_ff else []):
+            q = p + f'mlp.{e}.'
+            out[q + 'gate'], out[q + 'up'], out[q + 'down'] = (ff, W), (ff, W), (W, ff)
+        if s.shared_gate:
+            out[p + 'mlp.shared.sg'] = (1, W)
+    return out
+
+
+def _rotation(i: int, m: dict, s: LayerSpec):
+    """rot: {"base", "dims"} of a mixer's config -> the spec (absent: no rotation; without dims: the whole head)"""
+    rot = m.get('rot') or {}
+    s.rot_dims = int(rot.get('dims', s.dim)) if rot else 0
+    s.rot_base = float(rot.get('base', 10000.0))
+    if s.rot_dims % 2 or not 0 <= s.rot_dims <= s.dim:
+        raise ValueError(f'layer {i}: rot.dims must be even and at most dim')
+
+
+def _roravik_layer(i: int, L: dict, shapes: dict) -> LayerSpec:
+    m, mlp, kind = L['mixer'], L.get('mlp'), L['type']
+    s = LayerSpec(both_norms=True)
+    if kind == 'retention':
+        s.mixer, s.heads, s.dim = MIXER_RETENTION, int(m['heads']), int(m['dim'])
+        s.kv_heads, s.vdim = s.heads, int(m.get('vdim', s.dim))
+        d = m['decay']
+        s.decay = tuple(float(v) for v in d) if isinstance(d, (list, tuple)) else (float(d),) * s.heads
+        if len(s.decay) != s.heads:
+            raise ValueError(f'layer {i}: one decay per head')
+        _rotation(i, m, s)
+    elif kind == 'parallel':
+        a, b = m['left'], m['right']
+        s.mixer, s.heads, s.dim = MIXER_PARALLEL, int(a['heads']), int(a['dim'])
+        s.kv_heads, s.vdim = int(a.get('kv_heads', s.heads)), int(a.get('vdim', s.dim))
+        s.scale = float(a['scale']) if 'scale' in a else s.dim ** -0.5
+        s.softcap, s.sink = float(a.get('softcap') or 0.0), True
+        s.window = int((a.get('mask') or {}).get('size') or 0)
+        conv = shapes.get(f'l{i}.mix.left.q.conv')
+        s.conv_taps = int(conv[1]) if conv else int(a.get('conv') or 0)
+        _rotation(i, a, s)
+        s.r_heads, s.r_dim = int(b['heads']), int(b['dim'])
+        s.r_kv_heads, s.r_vdim = s.r_heads, s.r_dim
+        w1 = shapes.get(f'l{i}.mix.right.w1')     # the inner size of the decay projection is the tensor's own
+        s.decay_rank = int(w1[0]) if w1 else int(b.get('decay_rank', 0) or max(1, min(64, s.r_dim // 2)))
+        s.left_scale, s.right_scale = float(m.get('left_scale', 1.0)), float(m.get('right_scale', 1.0))
+    else:
+        raise NotImplementedError(f'layer {i}: mixer {kind!r}')
+    if mlp is None:
+        return s
+    if mlp.get('kind') == 'dense':
+        s.mlp, s.ff, s.act, s.act_limit, s.act_alpha = MLP_GATED, int(mlp['ff']), ACT_CLAMPED, float(mlp['limit']), 1.702
+    elif mlp.get('kind') == 'moe':
+        r, shared = mlp['router'], mlp.get('shared') or {}
+        s.mlp, s.ff, s.act, s.experts, s.top = MLP_MOE, int(mlp['expert']['ff']), ACT_SILU, int(r['experts']), int(r['top'])
+        g = r.get('groups') or {}
+        s.group_count, s.group_keep = int(g.get('count', 1)), int(g.get('keep', g.get('count', 1)))
+        s.router_correction = s.router_renorm = True
+        s.shared_ff = int(shared.get('ff', 0))
+        s.shared_gate = s.shared_ff > 0
+        if s.experts % s.group_count or not 1 <= s.group_keep <= s.group_count or s.top > s.experts // s.group_count * s.group_keep:
+            raise ValueError(f'layer {i}: the groups must divide the experts and the kept ones must hold at least `top` of them')
+    else:
+        raise NotImplementedError(f'layer {i}: feed-forward kind {mlp.get("kind")!r}')
+    return s
+
+
+def _loop_runs(c: dict, own: list):
+    """`own` (one spec per layer) with config 'loop' unrolled -> (layer runs, checkpoint prefix of every run, passes): a run of a later pass
+    names the first one's tensors in weights_of, the first run of a pass carries its number in loop_pass"""
+    import copy
+    loop = c.get('loop') or {}
+    start, stop, times = int(loop.get('start', 0)), int(loop.get('stop', 0)), int(loop.get('times', 0))
+    if not 0 <= start <= stop <= len(own):
+        raise ValueError('loop: 0 <= start <= stop <= layers')
+    if stop <= start or times < 1:
+        start = stop = times = 0
+    runs, names = [], []
+    first_run = {}      # layer -> its first run (the one that owns the tensors)
+    order = list(range(start)) + [i for _ in range(times) for i in range(start, stop)] + list(range(stop, len(own)))
+    seen_pass = 0
+    for at, i in enumerate(order):
+        s = copy.copy(own[i])
+        if times and i == start and start <= at < start + times * (stop - start):
+            s.loop_pass, seen_pass = seen_pass, seen_pass + 1
+        if i in first_run:
+            s.weights_of = first_run[i]
+        else:
+            first_run[i] = len(runs)
+        runs.append(s)
+        names.append(f'l{i}.')
+    return runs, names, times
+
+
+def _roravik(c: dict, shapes: dict | None = None) -> LayeredConfig:
+    """Roravik: blocks x += N(mixer(N x)); x += N(ff(N x)) with RMS norms whose weights are stored around zero.  Mixers: retention (linear
+    attention, one fixed decay per head, rotated queries and keys, a silu gate), or a parallel pair -- windowed grouped-query attention with
+    convolved projections, rotation, capped scores and a sink per head, beside a time mixer (a decay per token and key channel, every
+    projection reads its own mix of a token and its predecessor, a bonus for the current token) -- whose results are summed with weights.
+    Feed-forwards: a clamped gated unit, or sigmoid-routed gated-silu experts chosen inside the best groups by corrected scores, plus a
+    gated shared expert.  A range of layers may run several times on the same weights; the embedding output joins the stream ahead of
+    every pass but the first.  Tied embedding, scaled on the way in; capped logits.  `shapes` ({tensor name: shape} of the checkpoint)
+    settles the sizes the config leaves to the tensors."""
+    runs, names, times = _loop_runs(c, [_roravik_layer(i, L, shapes or {}) for i, L in enumerate(c['layers'])])
+    return LayeredConfig(arch='Roravik', width=int(c['width']), vocab=int(c['vocab']), layers=runs, norm_eps=float(c['norm']['eps']),
+                         norm_offset=1.0, residual_mult=1.0, logit_scale=1.0, eos_token_id=c.get('eos_token_id'),
+                         embed_scale=float((c.get('embedding') or {}).get('scale', 1.0)), logit_softcap=float(c.get('logit_softcap') or 0.0),
+                         loop_add=times > 1, tied_head=True, names=names)
 
 
 def _sanozen_layer(i: int, L: dict, specs: list) -> LayerSpec:
@@ -495,26 +656,7 @@ def _bedenex(c: dict) -> LayeredConfig:
     part cached per token, a sink logit per head).  Feed-forwards: gated GELU, or a sigmoid-routed mixture of gated SiLU experts whose
     scores scale the experts' inputs.  A range of layers may run several times in a row on the same weights (every run has its own cache);
     each pass starts from loop.in [x | embedding output] + loop.step[pass]."""
-    import copy
-    own = [_bedenex_layer(i, L) for i, L in enumerate(c['layers'])]
-    loop = c.get('loop') or {}
-    start, stop, times = int(loop.get('start', 0)), int(loop.get('stop', 0)), int(loop.get('times', 0))
-    if stop <= start or times < 1:
-        start = stop = times = 0
-    runs, names = [], []
-    first_run = {}      # layer -> its first run (the one that owns the tensors)
-    order = list(range(start)) + [i for _ in range(times) for i in range(start, stop)] + list(range(stop, len(own)))
-    seen_pass = 0
-    for i in order:
-        s = copy.copy(own[i])
-        if times and i == start:
-            s.loop_pass, seen_pass = seen_pass, seen_pass + 1
-        if i in first_run:
-            s.weights_of = first_run[i]
-        else:
-            first_run[i] = len(runs)
-        runs.append(s)
-        names.append(f'l{i}.')
+    runs, names, times = _loop_runs(c, [_bedenex_layer(i, L) for i, L in enumerate(c['layers'])])
     return LayeredConfig(arch='Bedenex', width=int(c['width']), vocab=int(c['vocab']), layers=runs, norm_eps=float(c['norm']['eps']),
                          norm_offset=0.0, residual_mult=1.0, logit_scale=1.0, eos_token_id=c.get('eos_token_id'), loop_times=times,
                          names=names)
@@ -547,8 +689,8 @@ def _fokonex(c: dict) -> LayeredConfig:
                          logit_scale=float(c['logit_scale']), eos_token_id=c.get('eos_token_id'))
 
 
-FAMILIES = {'Fokonex': _fokonex, 'Bedenex': _bedenex, 'Febivik': _febivik, 'Mededra': _mededra, 'Sanozen': _sanozen}
-NEEDS_SHAPES = {'Febivik', 'Mededra'}     # readers that take the checkpoint's tensor shapes as a second argument
+FAMILIES = {'Fokonex': _fokonex, 'Bedenex': _bedenex, 'Febivik': _febivik, 'Mededra': _mededra, 'Sanozen': _sanozen, 'Roravik': _roravik}
+NEEDS_SHAPES = {'Febivik', 'Mededra', 'Roravik'}     # readers that take the checkpoint's tensor shapes as a second argument
 
 
 def is_layered(model_path: str) -> bool:
