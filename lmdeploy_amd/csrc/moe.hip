@@ -577,28 +577,36 @@ int launch_moe_gather(void* xs, int lds, const void* x, int ldx, int elem_bytes,
     return 0;
 }
 
-// resid[t] += gate(t) * sum_j (weighted ? w[t][j] : 1) * y[en2f[j][t]], gate(t)[i] = sigmoid(gate[t][i] + gate_bias[i]) (gate == nullptr: 1)
+// resid[t] += gate(t) * sum_j (weighted ? w[t][j] : 1) * y[en2f[j][t]], gate(t)[i] = sigmoid(gate[t][i] + gate_bias[i]) (gate == nullptr: 1);
+// VEC neighbouring channels per thread (VEC = 4: H is a multiple of four)
+template<int VEC>
 __global__ void moe_combine_f32_kernel(float* __restrict__ resid, const float* __restrict__ y, const float* __restrict__ w, const int* __restrict__ en2f,
                                        const float* __restrict__ gate, int ldg, const float* __restrict__ gate_bias, int Tn, int H, int k, int weighted,
                                        int overwrite, const float* __restrict__ add, const float* __restrict__ add_gate, int ld_ag)
 {
-    const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+    typedef float VF __attribute__((ext_vector_type(VEC)));
+    const size_t i = ((size_t)blockIdx.x * blockDim.x + threadIdx.x) * VEC;
     if (i >= (size_t)Tn * H) {
         return;
     }
     const int t = (int)(i / H), c = (int)(i % H);
-    float     s = 0.f;
+    VF        s = 0.f;
     for (int j = 0; j < k; ++j) {
-        const float v = y[(size_t)en2f[(size_t)j * Tn + t] * H + c];
+        const VF v = *(const VF*)(y + (size_t)en2f[(size_t)j * Tn + t] * H + c);
         s += weighted ? w[(size_t)t * k + j] * v : v;
     }
     if (gate) {
-        s = s / (1.f + expf(-(gate[(size_t)t * ldg + c] + gate_bias[c])));
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) {
+            s[e] = s[e] / (1.f + expf(-(gate[(size_t)t * ldg + c + e] + gate_bias[c + e])));
+        }
     }
     if (add) {
-        s = (add_gate ? add[i] / (1.f + expf(-add_gate[(size_t)t * ld_ag])) : add[i]) + s;
+        const VF a = *(const VF*)(add + i);
+        s = (add_gate ? a / (1.f + expf(-add_gate[(size_t)t * ld_ag])) : a) + s;
     }
-    resid[i] = overwrite ? s : resid[i] + s;
+    VF* out = (VF*)(resid + i);
+    *out    = overwrite ? s : *out + s;
 }
 
 int launch_moe_combine_f32(float* resid, const float* y, const float* w, const int* en2f, const float* gate, int ldg, const float* gate_bias, int T,
@@ -609,7 +617,12 @@ int launch_moe_combine_f32(float* resid, const float* y, const float* w, const i
     if (total == 0) {
         return 0;
     }
-    moe_combine_f32_kernel<<<(total + 255) / 256, 256, 0, st>>>(resid, y, w, en2f, gate, ldg, gate_bias, T, H, k, weighted, overwrite, add, add_gate, ld_add_gate);
+    if (H % 4 == 0) {
+        moe_combine_f32_kernel<4><<<(total / 4 + 255) / 256, 256, 0, st>>>(resid, y, w, en2f, gate, ldg, gate_bias, T, H, k, weighted, overwrite, add, add_gate, ld_add_gate);
+    }
+    else {
+        moe_combine_f32_kernel<1><<<(total + 255) / 256, 256, 0, st>>>(resid, y, w, en2f, gate, ldg, gate_bias, T, H, k, weighted, overwrite, add, add_gate, ld_add_gate);
+    }
     TM_HIP_CHECK(hipGetLastError());
     return 0;
 }

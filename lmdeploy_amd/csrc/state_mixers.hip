@@ -978,7 +978,8 @@ int launch_short_conv(float* y, int ldy, const float* x, int ldx, int x_col, con
 
 // y[row][g * n + i] = x[row][g * n + i] / sqrt(mean_i(x[row][g, :]^2) + eps) * w[g * n + i] * sigmoid(gate[row][g * n + i]):
 // the output norm of the state mixers over groups of n channels (all heads together, or head by head) and their sigmoid gate (gate == nullptr: none).
-// One workgroup per row: a single group is reduced by the whole workgroup, several groups are dealt to its four waves.
+// One workgroup per row: a single group is reduced by the whole workgroup, several groups are dealt to its four waves (and to grid y
+// workgroups where the rows are too few to fill the device).
 template<class T>
 __global__ __launch_bounds__(256) void gated_group_norm_kernel(T* __restrict__ y, int ldy, const float* __restrict__ x, int ldx,
                                                                const float* __restrict__ w, const float* __restrict__ gate, int ldg, int groups,
@@ -1011,7 +1012,7 @@ __global__ __launch_bounds__(256) void gated_group_norm_kernel(T* __restrict__ y
         }
         return;
     }
-    for (int g = wave; g < groups; g += 4) {
+    for (int g = blockIdx.y * 4 + wave; g < groups; g += gridDim.y * 4) {
         const float* xg = xr + (size_t)g * n;
         float        ss = 0.f;
         for (int i = lane; i < n; i += 64) {
@@ -1032,11 +1033,12 @@ int launch_gated_group_norm(void* y, int ldy, int out_elem_bytes, const float* x
     if (rows == 0) {
         return 0;
     }
+    const dim3 grid(rows, groups > 4 && rows <= 256 ? (groups + 3) / 4 : 1);
     if (out_elem_bytes == 2) {
-        gated_group_norm_kernel<__bf16><<<rows, 256, 0, st>>>((__bf16*)y, ldy, x, ldx, w, gate, ldg, groups, n, eps, silu, mult);
+        gated_group_norm_kernel<__bf16><<<grid, 256, 0, st>>>((__bf16*)y, ldy, x, ldx, w, gate, ldg, groups, n, eps, silu, mult);
     }
     else {
-        gated_group_norm_kernel<float><<<rows, 256, 0, st>>>((float*)y, ldy, x, ldx, w, gate, ldg, groups, n, eps, silu, mult);
+        gated_group_norm_kernel<float><<<grid, 256, 0, st>>>((float*)y, ldy, x, ldx, w, gate, ldg, groups, n, eps, silu, mult);
     }
     TM_HIP_CHECK(hipGetLastError());
     return 0;

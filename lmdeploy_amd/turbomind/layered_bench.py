@@ -24,6 +24,11 @@ width, heads, layer count and vocabulary.
 cache; a forget-gate state mixer; PolyNorm feed-forward; token-side input; average over the depth) beside the closest model the engine
 serves -- the Bedenex blocks above (latent attention in the same latent space, fused fp32 projections) -- at equal width, heads, layer
 count and vocabulary and a feed-forward of the same parameter count.
+
+`bench.py --layered --layered-design roravik`: Roravik blocks (retention; the parallel pair of a convolved windowed attention and a time
+mixer; clamped and routed gated feed-forwards with a gated shared expert; norms on both sides of the sublayers) beside the closest model
+the engine serves -- the Febivik blocks above (lightning and delta-rule state mixers, windowed attention, routed experts with a shared
+one) -- at equal width, heads, layer count, vocabulary and active feed-forward parameters.
 """
 from __future__ import annotations
 
@@ -265,6 +270,62 @@ def _sanozen_decode_bytes(s, batch, ctx):
     return out
 
 
+RORAVIK = dict(window=2048, conv=4, decay_rank=64, experts=8, top=2)
+
+
+def _roravik_expert_ff(s):
+    return s['inter'] // 48 * 16      # three matrices of a third of the dense size, in sixteens
+
+
+def roravik_config(s) -> dict:
+    """config.json of the benchmark model: [retention + dense, parallel + experts, retention + experts, parallel + experts] repeated, head size
+    128 everywhere; the dense feed-forward has the size's own `inter`, experts and the shared expert a third of it, two experts per token"""
+    b, H = RORAVIK, s['heads']
+    rot = {'base': 10000.0, 'dims': 128}
+    ret = {'heads': H, 'dim': 128, 'vdim': 128, 'decay': [1.0 - 2.0 ** -(5 + 5 * h / max(1, H - 1)) for h in range(H)], 'rot': rot}
+    left = {'heads': H, 'kv_heads': s['kv_heads'], 'dim': 128, 'vdim': 128, 'conv': b['conv'], 'scale': 128 ** -0.5, 'softcap': 30.0,
+            'mask': {'size': b['window']}, 'rot': rot}
+    par = {'left': left, 'right': {'heads': H, 'dim': 128, 'decay_rank': b['decay_rank']}, 'left_scale': 0.75, 'right_scale': 1.25}
+    ff = _roravik_expert_ff(s)
+    dense = {'kind': 'dense', 'ff': s['inter'], 'limit': 7.0}
+    moe = {'kind': 'moe', 'expert': {'ff': ff}, 'router': {'experts': b['experts'], 'top': b['top'], 'groups': {'count': 4, 'keep': 2}},
+           'shared': {'ff': ff}}
+    four = [{'type': 'retention', 'mixer': ret, 'mlp': dense}, {'type': 'parallel', 'mixer': par, 'mlp': moe},
+            {'type': 'retention', 'mixer': ret, 'mlp': moe}, {'type': 'parallel', 'mixer': par, 'mlp': moe}]
+    return {'architecture': 'Roravik', 'width': s['width'], 'vocab': s['vocab'], 'norm': {'eps': 1e-5}, 'embedding': {'scale': 1.0},
+            'logit_softcap': 30.0, 'layers': [four[i % 4] for i in range(s['layers'])]}
+
+
+def _roravik_engine(s, batch, session_len, max_prefill):
+    from . import layered
+    cfg = layered.FAMILIES['Roravik'](roravik_config(s))
+    eng = layered.LayeredEngine(cfg, dtype='bfloat16', max_batch_size=batch, session_len=session_len, max_prefill_token_num=max_prefill)
+    eng.init_synthetic(seed=1)
+    eng.start()
+    return eng
+
+
+def _roravik_decode_bytes(s, batch, ctx):
+    """bytes each category of ONE decode step must move: every weight that takes part once (all experts), the cache entries inside the
+    window once per sequence, and every recurrent state read and written once (fp32)"""
+    b, W, H, G, V = RORAVIK, s['width'], s['heads'], s['kv_heads'], s['vocab']
+    out = dict(gemm_qkv=0, attention=0, gemm_o=0, gemm_gate_up=0, gemm_down=0, lm_head=2 * W * V)
+    for i in range(s['layers']):
+        moe, state = i % 4 != 0, batch * H * 128 * 128 * 4 * 2
+        if i % 2 == 0:
+            out['gemm_qkv'] += 2 * W * 4 * H * 128
+            out['attention'] += state
+            out['gemm_o'] += 2 * W * H * 128
+        else:
+            out['gemm_qkv'] += 2 * W * ((H + 2 * G) * 128 + 4 * H * 128) + 2 * b['decay_rank'] * (W + H * 128)
+            out['attention'] += state + 2 * batch * 2 * G * 128 * min(ctx, b['window'])
+            out['gemm_o'] += 2 * 2 * W * H * 128
+        n = (b['experts'] + 1) * _roravik_expert_ff(s) if moe else s['inter']
+        out['gemm_gate_up'] += 2 * W * 2 * n + (2 * W * (b['experts'] + 1) if moe else 0)
+        out['gemm_down'] += 2 * W * n
+    return out
+
+
 def _measure(eng, vocab, batch, prompt_len, steps, warmup, prefill_seqs):
     rng = np.random.default_rng(0)
     out = {}
@@ -315,7 +376,8 @@ def run(steps: int, warmup: int, batch: int, prompt_len: int, sizes=None, design
             'bedenex': (('bedenex_bf16', _bedenex_engine), ('fokonex_bf16', _fokonex_engine)),
             'febivik': (('febivik_bf16', _febivik_engine), ('bedenex_bf16', _bedenex_engine)),
             'mededra': (('mededra_bf16', _mededra_engine), ('febivik_bf16', _febivik_engine)),
-            'sanozen': (('sanozen_bf16', _sanozen_engine), ('bedenex_bf16', _bedenex_engine))}[design]
+            'sanozen': (('sanozen_bf16', _sanozen_engine), ('bedenex_bf16', _bedenex_engine)),
+            'roravik': (('roravik_bf16', _roravik_engine), ('febivik_bf16', _febivik_engine))}[design]
     if only_first:
         pair = pair[:1]
     for name in (sizes or SIZES):
@@ -327,7 +389,7 @@ def run(steps: int, warmup: int, batch: int, prompt_len: int, sizes=None, design
             eng = make(s, batch, session_len, 8192)
             m = _measure(eng, s['vocab'], batch, prompt_len, steps, warmup, prefill_seqs)
             ctx = prompt_len + warmup + steps // 2
-            need = _sanozen_decode_bytes(s, batch, ctx) if kind == 'sanozen_bf16' else _mededra_decode_bytes(s, batch, ctx) if kind == 'mededra_bf16' else _febivik_decode_bytes(s, batch, ctx) if kind == 'febivik_bf16' else \
+            need = _roravik_decode_bytes(s, batch, ctx) if kind == 'roravik_bf16' else _sanozen_decode_bytes(s, batch, ctx) if kind == 'sanozen_bf16' else _mededra_decode_bytes(s, batch, ctx) if kind == 'mededra_bf16' else _febivik_decode_bytes(s, batch, ctx) if kind == 'febivik_bf16' else \
                 _bedenex_decode_bytes(s, batch, ctx) if kind == 'bedenex_bf16' else _decode_bytes(s, batch, ctx, kind == 'fokonex_bf16')
             m['decode_hbm_roofline_fraction'] = {k: round(need[k] / HBM_BYTES_PER_S / (m['decode_categories_ms'][k] * 1e-3), 4)
                                                  for k in need if m['decode_categories_ms'].get(k)}
