@@ -2,9 +2,9 @@
 batching -- nothing here is shared with the engine.  `cfg` is the parsed config.json, `w` maps tensor names to float64 arrays.
 
 A block has a norm ahead of each sublayer and one behind it: x += N1b(mixer(N1 x)); x += N2b(ff(N2 x)), N an RMS norm whose weight is
-stored around zero.  A range of layers runs several times on the same weights; ahead of every pass but the first the embedding output is
-added to the stream.
-Mixers: `retention` -- a state per head with one fixed decay, S_t = g S_(t-1) + k_t v_t^T, o_t = S_t^T q_t, rotated queries and keys, unit-RMS
+stored around zero.  A range of layers runs several times on the same weights; from the second pass on the stream is joined by the
+embedding output where the pass begins.
+Mixers: `retention` -- a state per head with one fixed decay, S <- g S + k v^T, o = S^T q, rotated queries and keys, unit-RMS
 heads, a silu gate.  `parallel` -- left: windowed grouped-query attention with convolved projections, rotation, capped scores and a sink in
 the soft-max denominator; right: a state per head with a decay per token and key channel, every projection reading its own mix of the
 token and its predecessor, a bonus for the current token; the result is a weighted sum of both.
@@ -49,7 +49,7 @@ def rotate_half(x, pos, dims, base):
 
 
 def short_conv(u, w):
-    """u [T, C], w [C, taps]: y_t = sum_j w[:, j] u_(t - taps + 1 + j), zeros ahead of the sequence"""
+    """u [T, C], w [C, n] -> out[t] = w[:, n-1] u[t] + w[:, n-2] u[t-1] + ...; rows ahead of the sequence count as zero"""
     taps = w.shape[1]
     pad = np.concatenate([np.zeros((taps - 1, u.shape[1])), u])
     return sum(w[:, j] * pad[j:j + len(u)] for j in range(taps))
@@ -111,7 +111,8 @@ def previous(h):
 
 
 def bonus_recurrence(r, k, v, decay, u, state=None):
-    """r, k, decay [T, d], v [T, dv], u [d]: o_t = (S + diag(u) k_t v_t^T)^T r_t with the state BEFORE token t; S <- diag(decay_t) S + k_t v_t^T"""
+    """r, k, decay [T, d], v [T, dv], u [d]: the token reads the state of its
+    predecessors plus its own pair weighted by u, o = r^T S + (r . (u k)) v; then S <- diag(decay) S + k v^T"""
     S = np.zeros((r.shape[1], v.shape[1])) if state is None else state.copy()
     o = np.zeros((len(r), v.shape[1]))
     for t in range(len(r)):
